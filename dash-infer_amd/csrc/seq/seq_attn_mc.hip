@@ -1,6 +1,6 @@
 // seq_attn_mc.hip -- windowed sink-softmax attention over the paged latent cache on the matrix cores (bf16 cache).
 //
-// All heads of a sequence share the cached latent rows C [keys, R]: they are keys AND values.  A workgroup owns 64
+// All heads of a sequence share the cached latent rows C [keys, R]: they are keys AND (their first RV elements) values.  A workgroup owns 64
 // consecutive (row, head) pairs of one portion -- 16 per wave -- and walks the key tiles of 32 cached rows its pairs can
 // see.  Per tile: S^T = C . Q^T (A = the tile's rows as they lie in LDS, B = the wave's query fragments, held in registers
 // for the whole walk), mask + running softmax on the accumulator lanes (a pair's 32 scores sit in the four 16-lane groups
@@ -20,7 +20,7 @@ struct McArgs {
   void* const* spans; int span_stride, span_len;
   const void* sink; int wdt;
   const int32_t* tok_pos; const int32_t* ent_slot; const int32_t* ent_row0; const int32_t* ent_count;
-  int H, R, window; float scale;
+  int H, R, RV, window; float scale;   // RV: the row's first RV elements are the value (multiple of 16)
   float* ws; int rows_total;
 };
 
@@ -28,13 +28,13 @@ __device__ __forceinline__ f32x4_t mfma_bf16x(const u32x4_t& a, const u32x4_t& b
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
-template <int RMAX>
+template <int RMAX, int RVMAX>
 __global__ __launch_bounds__(256) void latent_attn_mc_kernel(McArgs a) {
-  constexpr int KS = RMAX / 32, DT = RMAX / 16, UN = RMAX / 64;
+  constexpr int KS = RMAX / 32, DT = RVMAX / 16, UN = RMAX / 64;
   constexpr bool PREFETCH = RMAX <= 256;  // the widest rows leave no registers for a tile in flight
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int e = blockIdx.y, split = blockIdx.z, nsplit = gridDim.z;
-  const int H = a.H, R = a.R;
+  const int H = a.H, R = a.R, RV = a.RV;
   const int cnt = a.ent_count[e], row0 = a.ent_row0[e];
   const int nrows = cnt * H, r0 = blockIdx.x * 64;
   if (r0 >= nrows) return;
@@ -154,7 +154,7 @@ __global__ __launch_bounds__(256) void latent_attn_mc_kernel(McArgs a) {
     const unsigned char* tr0 = smem + (kb * 4 + (ni >> 2)) * pitchb + (ni & 3) * 8;
 #pragma unroll
     for (int t = 0; t < DT; ++t) {
-      if (t * 16 < R) {
+      if (t * 16 < RV) {
         const u32x2_t lo2 = lds_read_tr16(tr0 + t * 32);
         const u32x2_t hi2 = lds_read_tr16(tr0 + t * 32 + 16 * pitchb);
         const u32x4_t vf = {lo2[0], lo2[1], hi2[0], hi2[1]};
@@ -167,32 +167,32 @@ __global__ __launch_bounds__(256) void latent_attn_mc_kernel(McArgs a) {
   if (!row_ok) return;
   if (nsplit == 1) {
     const float inv = 1.f / l;
-    float* o = a.out + (size_t)(row0 + tq) * a.ldo + (size_t)h * R + kb * 4;
+    float* o = a.out + (size_t)(row0 + tq) * a.ldo + (size_t)h * RV + kb * 4;
 #pragma unroll
     for (int t = 0; t < DT; ++t)
-      if (t * 16 < R) *reinterpret_cast<f32x4_t*>(o + t * 16) = f32x4_t{oacc[t][0] * inv, oacc[t][1] * inv, oacc[t][2] * inv, oacc[t][3] * inv};
+      if (t * 16 < RV) *reinterpret_cast<f32x4_t*>(o + t * 16) = f32x4_t{oacc[t][0] * inv, oacc[t][1] * inv, oacc[t][2] * inv, oacc[t][3] * inv};
   } else {
-    float* o = a.ws + ((size_t)split * a.rows_total + (size_t)(row0 + tq) * H + h) * (R + 4);
+    float* o = a.ws + ((size_t)split * a.rows_total + (size_t)(row0 + tq) * H + h) * (RV + 4);
 #pragma unroll
     for (int t = 0; t < DT; ++t)
-      if (t * 16 < R) *reinterpret_cast<f32x4_t*>(o + t * 16 + kb * 4) = oacc[t];
-    if (kb == 0) { o[R] = m; o[R + 1] = l; }
+      if (t * 16 < RV) *reinterpret_cast<f32x4_t*>(o + t * 16 + kb * 4) = oacc[t];
+    if (kb == 0) { o[RV] = m; o[RV + 1] = l; }
   }
 }
 
 __global__ __launch_bounds__(256) void latent_attn_merge_kernel(float* __restrict__ out, long ldo, const float* __restrict__ ws, int nsplit,
-                                                                int rows_total, int H, int R) {
+                                                                int rows_total, int H, int RV) {
   __shared__ float wgt[1024];
   __shared__ float red[4];
   const int g = blockIdx.x, t = g / H, h = g - t * H;
-  const size_t rec = (size_t)R + 4, stride = (size_t)rows_total * rec;
+  const size_t rec = (size_t)RV + 4, stride = (size_t)rows_total * rec;
   const float* base = ws + (size_t)g * rec;
   float mloc[4], lloc[4], mx = -INFINITY;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int s = threadIdx.x + i * 256;
-    mloc[i] = s < nsplit ? base[s * stride + R] : -INFINITY;
-    lloc[i] = s < nsplit ? base[s * stride + R + 1] : 0.f;
+    mloc[i] = s < nsplit ? base[s * stride + RV] : -INFINITY;
+    lloc[i] = s < nsplit ? base[s * stride + RV + 1] : 0.f;
     mx = fmaxf(mx, mloc[i]);
   }
   mx = wave_max(mx);
@@ -209,11 +209,11 @@ __global__ __launch_bounds__(256) void latent_attn_merge_kernel(float* __restric
   }
   den = block256_sum(den, red);      // (its barriers publish wgt)
   const float inv = 1.f / den;
-  for (int r = threadIdx.x; r < R; r += 256) {
+  for (int r = threadIdx.x; r < RV; r += 256) {
     float acc = 0.f;
 #pragma unroll 8
     for (int s = 0; s < nsplit; ++s) acc = __builtin_fmaf(wgt[s], base[s * stride + r], acc);
-    out[(size_t)t * ldo + (size_t)h * R + r] = acc * inv;
+    out[(size_t)t * ldo + (size_t)h * RV + r] = acc * inv;
   }
 }
 
@@ -225,38 +225,41 @@ using namespace dihip;
 extern "C" {
 
 int dihip_latent_window_attn_mc_supported(int R, int span_len, int cache_dtype) {
-  return cache_dtype == DIHIP_BF16 && R % 32 == 0 && R >= 32 && R <= 512 && span_len % 32 == 0;
+  return cache_dtype == DIHIP_BF16 && R % 32 == 0 && R >= 32 && R <= 640 && span_len % 32 == 0;
 }
 
-size_t dihip_latent_window_attn_mc_workspace_bytes(int T, int H, int R, int nsplit) {
-  return nsplit > 1 ? (size_t)nsplit * T * H * (R + 4) * sizeof(float) : 0;
+size_t dihip_latent_window_attn_mc_workspace_bytes(int T, int H, int RV, int nsplit) {
+  return nsplit > 1 ? (size_t)nsplit * T * H * (RV + 4) * sizeof(float) : 0;
 }
 
 int dihip_latent_window_attn_mc(void* stream, float* out, long ldo, const float* q, long ldq, void* const* spans, int span_stride,
                                 int span_len, const void* sink, int w_dtype, const int32_t* tok_pos, const int32_t* ent_slot,
-                                const int32_t* ent_row0, const int32_t* ent_count, int E, int max_count, int T, int H, int R, int window,
+                                const int32_t* ent_row0, const int32_t* ent_count, int E, int max_count, int T, int H, int R, int RV, int window,
                                 float scale, int nsplit, void* ws, size_t ws_bytes) {
   DIHIP_REQUIRE(dihip_latent_window_attn_mc_supported(R, span_len, DIHIP_BF16), DIHIP_PARAM_ERROR,
-                "latent_window_attn_mc: R %d (a multiple of 32 up to 512) / span_len %d (a multiple of 32) not served", R, span_len);
+                "latent_window_attn_mc: R %d (a multiple of 32 up to 640) / span_len %d (a multiple of 32) not served", R, span_len);
+  DIHIP_REQUIRE(RV > 0 && RV <= R && RV <= 512 && RV % 16 == 0, DIHIP_PARAM_ERROR,
+                "latent_window_attn_mc: a value of %d elements (a multiple of 16 up to 512 inside the row) not served", RV);
   DIHIP_REQUIRE(E >= 0 && T >= 0 && H > 0 && max_count >= 0 && out && q && spans && tok_pos && ent_slot && ent_row0 && ent_count &&
-                    span_stride > 0 && ldo >= (long)H * R && ldq >= (long)H * R && ldo % 4 == 0 && ldq % 4 == 0 && seq_dtype_ok(w_dtype),
+                    span_stride > 0 && ldo >= (long)H * RV && ldq >= (long)H * R && ldo % 4 == 0 && ldq % 4 == 0 && seq_dtype_ok(w_dtype),
                 DIHIP_PARAM_ERROR, "latent_window_attn_mc: bad argument");
   DIHIP_REQUIRE((reinterpret_cast<uintptr_t>(out) & 15u) == 0 && (reinterpret_cast<uintptr_t>(q) & 15u) == 0, DIHIP_PARAM_ERROR,
                 "latent_window_attn_mc: q / out must be 16-byte aligned");
   DIHIP_REQUIRE(nsplit >= 1 && nsplit <= 1024 && E <= 65535, DIHIP_PARAM_ERROR, "latent_window_attn_mc: bad split / portion count");
-  DIHIP_REQUIRE(ws_bytes >= dihip_latent_window_attn_mc_workspace_bytes(T, H, R, nsplit) && (nsplit == 1 || ws), DIHIP_PARAM_ERROR,
+  DIHIP_REQUIRE(ws_bytes >= dihip_latent_window_attn_mc_workspace_bytes(T, H, RV, nsplit) && (nsplit == 1 || ws), DIHIP_PARAM_ERROR,
                 "latent_window_attn_mc: workspace too small");
   if (E == 0 || max_count == 0) return DIHIP_SUCCESS;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  McArgs a{out, ldo, q, ldq, spans, span_stride, span_len, sink, w_dtype, tok_pos, ent_slot, ent_row0, ent_count, H, R, window, scale,
+  McArgs a{out, ldo, q, ldq, spans, span_stride, span_len, sink, w_dtype, tok_pos, ent_slot, ent_row0, ent_count, H, R, RV, window, scale,
            (float*)ws, T * H};
   const dim3 grid((unsigned)(((long)max_count * H + 63) / 64), E, nsplit);
   const size_t lds = (size_t)32 * (R + 8) * 2;
-  if (R <= 64) hipLaunchKernelGGL(latent_attn_mc_kernel<64>, grid, dim3(256), lds, s, a);
-  else if (R <= 128) hipLaunchKernelGGL(latent_attn_mc_kernel<128>, grid, dim3(256), lds, s, a);
-  else if (R <= 256) hipLaunchKernelGGL(latent_attn_mc_kernel<256>, grid, dim3(256), lds, s, a);
-  else hipLaunchKernelGGL(latent_attn_mc_kernel<512>, grid, dim3(256), lds, s, a);
-  if (nsplit > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3(T * H), dim3(256), 0, s, out, ldo, (const float*)ws, nsplit, T * H, H, R);
+  if (R <= 64) hipLaunchKernelGGL((latent_attn_mc_kernel<64, 64>), grid, dim3(256), lds, s, a);
+  else if (R <= 128) hipLaunchKernelGGL((latent_attn_mc_kernel<128, 128>), grid, dim3(256), lds, s, a);
+  else if (R <= 256) hipLaunchKernelGGL((latent_attn_mc_kernel<256, 256>), grid, dim3(256), lds, s, a);
+  else if (R <= 512) hipLaunchKernelGGL((latent_attn_mc_kernel<512, 512>), grid, dim3(256), lds, s, a);
+  else hipLaunchKernelGGL((latent_attn_mc_kernel<640, 512>), grid, dim3(256), lds, s, a);
+  if (nsplit > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3(T * H), dim3(256), 0, s, out, ldo, (const float*)ws, nsplit, T * H, H, RV);
   return launch_status();
 }
 

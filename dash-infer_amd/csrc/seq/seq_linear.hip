@@ -15,6 +15,7 @@ struct LinArgs {
   void* y; long ldy, yg;
   const float* mul; long ldm;
   int T, N, K, act, act_lo, act_hi, ydt, round_ops;
+  int mul_group; float act_param;               // mul holds one number per group; the parameter of an activation that has one
   const int32_t* seg; const int32_t* row_map;   // segmented form: group g owns the output rows seg[g] .. seg[g + 1], row r reads x row row_map[r]
 };
 
@@ -28,9 +29,9 @@ __device__ __forceinline__ size_t lin_xrow(const LinArgs& a, int r) { return (si
 __device__ __forceinline__ void lin_epilogue(const LinArgs& a, int g, int t, int n, float v, int wdt) {
   if (a.bias) v += ld_any(a.bias, (size_t)g * a.N + n, wdt);
   const int col = g * a.N + n;
-  if (col >= a.act_lo && col < a.act_hi) v = apply_act(v, a.act);
+  if (col >= a.act_lo && col < a.act_hi) v = a.act == DIHIP_SEQ_ACT_SOFTCAP ? a.act_param * tanhf(v / a.act_param) : apply_act(v, a.act);
   const size_t o = (size_t)t * a.ldy + (size_t)g * a.yg + n;
-  if (a.mul) v *= a.mul[(size_t)t * a.ldm + (size_t)g * a.yg + n];
+  if (a.mul) v *= a.mul[(size_t)t * a.ldm + (a.mul_group ? (size_t)g : (size_t)g * a.yg + n)];
   st_any(a.y, o, a.ydt, v);
 }
 
@@ -351,18 +352,19 @@ using namespace dihip;
 
 static int linear_impl(void* stream, const void* x, int x_dtype, long ldx, long x_gstride, int x_groups, const void* w,
                        int w_dtype, const void* bias, void* y, int y_dtype, long ldy, long y_gstride, const float* mul,
-                       long ldm, int T, int N, int K, int groups, int act, int act_lo, int act_hi, int math,
+                       long ldm, int mul_group, int T, int N, int K, int groups, int act, int act_lo, int act_hi, float act_param, int math,
                        const int32_t* seg, const int32_t* row_map, int seg_max_rows) {
   DIHIP_REQUIRE(T >= 0 && N > 0 && K > 0 && groups > 0 && x_groups > 0, DIHIP_PARAM_ERROR, "linear: bad shape T %d N %d K %d groups %d", T, N, K, groups);
   DIHIP_REQUIRE(seq_dtype_ok(x_dtype) && seq_dtype_ok(w_dtype) && seq_dtype_ok(y_dtype), DIHIP_PARAM_ERROR, "linear: f32 / bf16 only");
   DIHIP_REQUIRE(x && w && y, DIHIP_PARAM_ERROR, "linear: null pointer");
-  DIHIP_REQUIRE(ldx >= K && ldy >= N && (!mul || ldm >= N), DIHIP_PARAM_ERROR, "linear: a row stride below the row length");
+  DIHIP_REQUIRE(ldx >= K && ldy >= N && (!mul || ldm >= (mul_group ? groups : N)), DIHIP_PARAM_ERROR, "linear: a row stride below the row length");
   DIHIP_REQUIRE(math == DIHIP_MATH_F32 || math == DIHIP_MATH_BF16 || math == DIHIP_MATH_F32_STREAM, DIHIP_PARAM_ERROR,
                 "linear: unknown math mode %d", math);
   DIHIP_REQUIRE(groups <= 65535, DIHIP_PARAM_ERROR, "linear: more than 65535 groups");
+  DIHIP_REQUIRE(act != DIHIP_SEQ_ACT_SOFTCAP || act_param > 0.f, DIHIP_PARAM_ERROR, "linear: a cap must be positive");
   if (T == 0) return DIHIP_SUCCESS;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  LinArgs a{x, ldx, x_gstride, x_groups, w, bias, y, ldy, y_gstride, mul, ldm, T, N, K, act, act_lo, act_hi, y_dtype, 0, seg, row_map};
+  LinArgs a{x, ldx, x_gstride, x_groups, w, bias, y, ldy, y_gstride, mul, ldm, T, N, K, act, act_lo, act_hi, y_dtype, 0, mul_group, act_param, seg, row_map};
   const int Tg = seg ? (seg_max_rows < T ? seg_max_rows : T) : T;   // the most rows one group can have
   const size_t xe = x_dtype == DIHIP_F32 ? 4 : 2;
   const bool vec = w_dtype == DIHIP_BF16 && K % 8 == 0 && aligned16(w) && aligned16(x) && (ldx * xe) % 16 == 0 &&
@@ -421,9 +423,10 @@ static int linear_impl(void* stream, const void* x, int x_dtype, long ldx, long 
 
 extern "C" int dihip_linear(void* stream, const void* x, int x_dtype, long ldx, long x_gstride, int x_groups, const void* w,
                             int w_dtype, const void* bias, void* y, int y_dtype, long ldy, long y_gstride, const float* mul,
-                            long ldm, int T, int N, int K, int groups, int act, int act_lo, int act_hi, int math) {
-  return linear_impl(stream, x, x_dtype, ldx, x_gstride, x_groups, w, w_dtype, bias, y, y_dtype, ldy, y_gstride, mul, ldm, T, N, K, groups,
-                     act, act_lo, act_hi, math, nullptr, nullptr, 0);
+                            long ldm, int mul_group, int T, int N, int K, int groups, int act, int act_lo, int act_hi,
+                            float act_param, int math) {
+  return linear_impl(stream, x, x_dtype, ldx, x_gstride, x_groups, w, w_dtype, bias, y, y_dtype, ldy, y_gstride, mul, ldm, mul_group, T, N, K, groups,
+                     act, act_lo, act_hi, act_param, math, nullptr, nullptr, 0);
 }
 
 extern "C" int dihip_linear_segmented(void* stream, const void* x, int x_dtype, long ldx, const void* w, int w_dtype, const void* bias,
@@ -431,6 +434,6 @@ extern "C" int dihip_linear_segmented(void* stream, const void* x, int x_dtype, 
                                       const int32_t* row_map, int seg_max_rows, int act, int math) {
   DIHIP_REQUIRE(seg && seg_max_rows >= 0, DIHIP_PARAM_ERROR, "linear_segmented: no segment table");
   if (seg_max_rows == 0) return DIHIP_SUCCESS;
-  return linear_impl(stream, x, x_dtype, ldx, 0, 1, w, w_dtype, bias, y, y_dtype, ldy, 0, nullptr, 0, R, N, K, groups, act, 0,
-                     act ? groups * N : 0, math, seg, row_map, seg_max_rows);
+  return linear_impl(stream, x, x_dtype, ldx, 0, 1, w, w_dtype, bias, y, y_dtype, ldy, 0, nullptr, 0, 0, R, N, K, groups, act, 0,
+                     act ? groups * N : 0, 0.f, math, seg, row_map, seg_max_rows);
 }

@@ -258,13 +258,13 @@ __global__ __launch_bounds__(256) void residual_norm_step_reg_kernel(float* x_ou
 // One workgroup per row, its 4 waves take the heads in turn.  A wave walks the row's window in chunks of 64 keys: lane j
 // scores key j (f32 dot over the R latent elements, r ascending), the chunk joins the running softmax (which starts at
 // the sink: maximum = sink, denominator = 1), then the lanes turn to the latent elements (lane l owns r = l, l + 64, ..)
-// and add the chunk's weighted rows.  Keys come from the cache only (the step's own rows were appended before).
-template <int CT, int RV>
+// and add the chunk's weighted rows (their first W elements: the value).  Keys come from the cache only (the step's own rows were appended before).
+template <int CT, int NV>
 __global__ __launch_bounds__(256) void latent_attn_kernel(float* __restrict__ out, long ldo, const float* __restrict__ q, long ldq,
                                                           void* const* __restrict__ spans, int span_stride, int span_len,
                                                           const void* __restrict__ sink, int wdt, const int32_t* __restrict__ tok_slot,
-                                                          const int32_t* __restrict__ tok_pos, int H, int R, int window, float scale) {
-  __shared__ float qs[4][RV * 64];
+                                                          const int32_t* __restrict__ tok_pos, int H, int R, int W, int window, float scale) {
+  __shared__ float qs[4][NV * 64];
   __shared__ float ps[4][64];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int pos = tok_pos[t];
@@ -280,9 +280,9 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(float* __restrict__ ou
     __syncthreads();
     float mx = -INFINITY, den = 0.f;
     if (sink) { mx = ld_any(sink, h < H ? h : 0, wdt); den = 1.f; }
-    float acc[RV];
+    float acc[NV];
 #pragma unroll
-    for (int v = 0; v < RV; ++v) acc[v] = 0.f;
+    for (int v = 0; v < NV; ++v) acc[v] = 0.f;
     for (int j0 = j_lo; j0 <= pos; j0 += 64) {  // the same trip count in every wave of the block
       const int j = j0 + lane;
       const bool valid = live && j <= pos;
@@ -298,7 +298,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(float* __restrict__ ou
       const float p = valid ? expf(s - mnew) : 0.f;
       den = den * corr + wave_sum(p);
 #pragma unroll
-      for (int v = 0; v < RV; ++v) acc[v] *= corr;
+      for (int v = 0; v < NV; ++v) acc[v] *= corr;
       mx = mnew;
       ps[wave][lane] = p;
       __syncthreads();
@@ -309,9 +309,9 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(float* __restrict__ ou
           const char* row = (const char*)tab[jk / span_len] + (size_t)(jk % span_len) * R * ES;
           const float pj = ps[wave][jj];
 #pragma unroll
-          for (int v = 0; v < RV; ++v) {
+          for (int v = 0; v < NV; ++v) {
             const int r = v * 64 + lane;
-            if (r < R) acc[v] = __builtin_fmaf(pj, load_ft<CT>(row, r), acc[v]);
+            if (r < W) acc[v] = __builtin_fmaf(pj, load_ft<CT>(row, r), acc[v]);
           }
         }
       }
@@ -319,9 +319,9 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(float* __restrict__ ou
     }
     if (live) {
 #pragma unroll
-      for (int v = 0; v < RV; ++v) {
+      for (int v = 0; v < NV; ++v) {
         const int r = v * 64 + lane;
-        if (r < R) out[(size_t)t * ldo + (size_t)h * R + r] = acc[v] / den;
+        if (r < W) out[(size_t)t * ldo + (size_t)h * W + r] = acc[v] / den;
       }
     }
   }
@@ -595,18 +595,18 @@ int dihip_add_dyt(void* stream, float* x_out, const float* x_in, const float* a,
 
 int dihip_latent_window_attn(void* stream, float* out, long ldo, const float* q, long ldq, void* const* spans, int span_stride,
                              int span_len, int cache_dtype, const void* sink, int w_dtype, const int32_t* tok_slot,
-                             const int32_t* tok_pos, int T, int H, int R, int window, float scale, int math) {
+                             const int32_t* tok_pos, int T, int H, int R, int RV, int window, float scale, int math) {
   DIHIP_REQUIRE(T >= 0 && H > 0 && R > 0 && out && q && spans && tok_slot && tok_pos && span_stride > 0 && span_len > 0 &&
-                    ldo >= (long)H * R && ldq >= (long)H * R && seq_dtype_ok(cache_dtype) && seq_dtype_ok(w_dtype),
+                    RV > 0 && RV <= R && ldo >= (long)H * RV && ldq >= (long)H * R && seq_dtype_ok(cache_dtype) && seq_dtype_ok(w_dtype),
                 DIHIP_PARAM_ERROR, "latent_window_attn: bad argument");
   DIHIP_REQUIRE(R <= 1024, DIHIP_EXCEED_LIMIT_ERROR, "latent_window_attn: latent rows of more than 1024 elements (%d)", R);
   (void)math;
   if (T == 0) return DIHIP_SUCCESS;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  auto go = [&](auto ct, auto rv) {
-    constexpr int CT = decltype(ct)::value, RV = decltype(rv)::value;
-    hipLaunchKernelGGL((latent_attn_kernel<CT, RV>), dim3(T), dim3(256), 0, s, out, ldo, q, ldq, spans, span_stride, span_len, sink,
-                       w_dtype, tok_slot, tok_pos, H, R, window, scale);
+  auto go = [&](auto ct, auto nv) {
+    constexpr int CT = decltype(ct)::value, NV = decltype(nv)::value;
+    hipLaunchKernelGGL((latent_attn_kernel<CT, NV>), dim3(T), dim3(256), 0, s, out, ldo, q, ldq, spans, span_stride, span_len, sink,
+                       w_dtype, tok_slot, tok_pos, H, R, RV, window, scale);
   };
   auto by_r = [&](auto ct) {
     if (R <= 64) go(ct, std::integral_constant<int, 1>{});

@@ -1,7 +1,6 @@
 // seq_moe.hip -- routing and glue of the mixture-of-experts feed-forward (the expert products are dihip_linear_segmented):
-//   moe_route      per token, f32: the `top` experts of largest router logit (ties: the lower index), weights = softmax over the
-//                  chosen logits alone; or (scoring 1) scores = softmax over ALL logits, the choice by score + a correction per
-//                  expert, weights = the chosen scores over their sum
+//   moe_route      per token, f32: the `top` experts of largest choice score and their weights (RouteRule below: scores = logits,
+//                  their softmax or their sigmoids; a correction for the choice alone; a choice limited to the best groups)
 //   moe_sort       the (token, choice) pairs grouped by expert in a fixed order: segment bounds per expert, the token each
 //                  sorted row reads, and where each pair went
 //   moe_glu        the experts' activation on [gate | up] rows (clamped sigmoid unit, or silu(gate) * up)
@@ -12,101 +11,157 @@
 namespace dihip {
 namespace {
 
-// One token's choice.  scoring 0: the `top` largest logits (ties: the lower index), weights = softmax over them alone.  scoring 1:
-// scores = softmax over all E logits, the choice by score + correction, weights = the chosen scores over their sum.  (Every logit
-// is read a few times: E is small and the row stays in cache.)
-template <int SCORING>
-__device__ __forceinline__ void route_token(const float* __restrict__ z, const void* __restrict__ corr, int cdt, int E, int top, int ngroups,
-                                            int keep, int (&bi)[32], float (&w)[32]) {
-  float zmax = -INFINITY, den = 1.f;
-  if (SCORING == 1) {
-    for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, z[e]);
-    den = 0.f;
-    for (int e = 0; e < E; ++e) den += expf(z[e] - zmax);
-  }
-  // group-limited choice: the experts form ngroups equal groups of neighbours, a group counts by its best expert, and only the
-  // experts of the `keep` best groups (ties: the lower index) can be chosen
-  uint32_t open_groups = 0xffffffffu;
-  const int gsz = ngroups > 1 ? E / ngroups : E;
-  if (ngroups > 1 && keep < ngroups) {
-    open_groups = 0u;
-    for (int k = 0; k < keep; ++k) {
-      float bv = -INFINITY;
-      int bg = -1;
-      for (int g = 0; g < ngroups; ++g) {
-        if (open_groups >> g & 1u) continue;
-        float gv = -INFINITY;
-        for (int e = g * gsz; e < (g + 1) * gsz; ++e) gv = fmaxf(gv, SCORING == 1 ? expf(z[e] - zmax) / den : z[e]);
-        if (bg < 0 || gv > bv) { bv = gv; bg = g; }
-      }
-      open_groups |= 1u << bg;
-    }
-  }
-  float sum = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float bv = -INFINITY, bs = 0.f;
-    int bx = -1;
-    for (int e = 0; e < E; ++e) {
-      bool used = false;
-      for (int j = 0; j < k; ++j) used |= bi[j] == e;
-      float v = z[e], sc = v;
-      if (SCORING == 1) {
-        sc = expf(v - zmax) / den;
-        v = sc + (corr ? ld_any(corr, e, cdt) : 0.f);
-      }
-      if (ngroups > 1 && !(open_groups >> (e / gsz) & 1u)) used = true;
-      if (!used && (bx < 0 || v > bv)) { bv = v; bx = e; bs = sc; }
-    }
-    w[k] = bs; bi[k] = bx;
-    sum += bs;
+// How a token's experts are chosen and weighted.
+//   scoring 0  scores = the logits, weights = softmax over the chosen logits alone
+//   scoring 1  scores = softmax over all E logits;  scoring 2  scores = sigmoid of every logit
+//              the choice goes by score + correction; weights = the chosen scores (over their sum with renorm) * factor
+//   ngroups    the experts form equal groups of neighbours; only experts of the `keep` best groups can be chosen (the others count as
+//              minus infinity).  A group counts by its largest score, or (group_top2) by the sum of its two largest choice scores
+// Ties: the lower index, in groups and experts.
+struct RouteRule {
+  const void* corr; int cdt;
+  int E, top, ngroups, keep, group_top2, renorm;
+  float factor;
+};
+
+// what one lane wrote to LDS is read by other lanes of the same wave
+__device__ __forceinline__ void wave_lds_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// One token per wave: lane l holds the experts l, l + 64, .. (NE of them), a choice is a maximum over the wave and the lowest index
+// that has it.  vals: E floats of LDS of this wave.  Afterwards lane k < top holds choice k and its weight.
+template <int SCORING, int NE>
+__device__ __forceinline__ void route_wave(const float* __restrict__ z, const RouteRule& r, float* vals, int& id, float& wt) {
+  constexpr float NONE = 16777216.f;     // an index beyond every expert
+  const int lane = threadIdx.x & 63;
+  float s[NE], c[NE];
+  float zmax = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = e < r.E ? z[e] : -INFINITY;
+    zmax = fmaxf(zmax, s[i]);
   }
   if (SCORING == 1) {
-    for (int k = 0; k < top; ++k) w[k] = w[k] / (sum + 1e-20f);
+    zmax = wave_max(zmax);
+    float den = 0.f;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      s[i] = lane + 64 * i < r.E ? expf(s[i] - zmax) : 0.f;
+      den += s[i];
+    }
+    den = wave_sum(den);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) s[i] /= den;
+  }
+  if (SCORING == 2) {
+#pragma unroll
+    for (int i = 0; i < NE; ++i) s[i] = 1.f / (1.f + expf(-s[i]));
+  }
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    c[i] = e < r.E ? s[i] + (r.corr ? ld_any(r.corr, e, r.cdt) : 0.f) : -INFINITY;
+  }
+  if (r.ngroups > 1 && r.keep < r.ngroups) {
+    const int gsz = r.E / r.ngroups;
+    wave_lds_sync();      // the token before is no longer read
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      if (lane + 64 * i < r.E) vals[lane + 64 * i] = r.group_top2 ? c[i] : s[i];
+    wave_lds_sync();
+    float gv = -INFINITY;
+    if (lane < r.ngroups) {
+      float m1 = -INFINITY, m2 = -INFINITY;
+      for (int e = lane * gsz; e < (lane + 1) * gsz; ++e) {
+        const float v = vals[e];
+        m2 = fmaxf(m2, fminf(m1, v));
+        m1 = fmaxf(m1, v);
+      }
+      gv = r.group_top2 && gsz > 1 ? m1 + m2 : m1;
+    }
+    unsigned long long open = 0ull;
+    for (int k = 0; k < r.keep; ++k) {
+      const float m = wave_max(gv);
+      const float g = wave_min(lane < r.ngroups && gv == m ? (float)lane : NONE);
+      open |= 1ull << min((int)g, r.ngroups - 1);
+      if (lane == (int)g) gv = -INFINITY;
+    }
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = lane + 64 * i;
+      if (e < r.E && !(open >> (e / gsz) & 1ull)) c[i] = -INFINITY;
+    }
+  }
+  id = 0;
+  wt = SCORING == 0 ? -INFINITY : 0.f;
+  for (int k = 0; k < r.top; ++k) {
+    float m = c[0];
+#pragma unroll
+    for (int i = 1; i < NE; ++i) m = fmaxf(m, c[i]);
+    m = wave_max(m);
+    float x = NONE;
+#pragma unroll
+    for (int i = NE - 1; i >= 0; --i)
+      if (lane + 64 * i < r.E && c[i] == m) x = (float)(lane + 64 * i);
+    const int best = min((int)wave_min(x), r.E - 1);
+    float sv = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      if (lane + 64 * i == best) { sv = s[i]; c[i] = -INFINITY; }
+    sv = wave_max(sv);
+    if (lane == k) { id = best; wt = sv; }
+  }
+  if (SCORING == 0) {
+    wt = expf(wt - __shfl(wt, 0));      // lanes past the choices: 0
+    wt = wt / wave_sum(wt);
   } else {
-    float d = 0.f;
-    const float m0 = w[0];
-    for (int k = 0; k < top; ++k) { w[k] = expf(w[k] - m0); d += w[k]; }
-    for (int k = 0; k < top; ++k) w[k] = w[k] / d;
+    if (r.renorm) wt = wt / (wave_sum(wt) + 1e-20f);
+    wt *= r.factor;
   }
 }
 
-template <int SCORING>
-__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, long ldl, const void* __restrict__ corr, int cdt,
-                                                        int32_t* __restrict__ ids, float* __restrict__ wts, int T, int E, int top, int ngroups, int keep) {
-  const int t = blockIdx.x * 256 + threadIdx.x;
+template <int SCORING, int NE>
+__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, long ldl, RouteRule r, int32_t* __restrict__ ids,
+                                                        float* __restrict__ wts, int T) {
+  extern __shared__ float route_vals[];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = blockIdx.x * 4 + wave;
   if (t >= T) return;
-  int bi[32];
-  float w[32];
-  route_token<SCORING>(logits + (size_t)t * ldl, corr, cdt, E, top, ngroups, keep, bi, w);
-  for (int k = 0; k < top; ++k) {
-    ids[(size_t)t * top + k] = bi[k];
-    wts[(size_t)t * top + k] = w[k];
+  int id;
+  float wt;
+  route_wave<SCORING, NE>(logits + (size_t)t * ldl, r, route_vals + (size_t)wave * r.E, id, wt);
+  if (lane < r.top) {
+    ids[(size_t)t * r.top + lane] = id;
+    wts[(size_t)t * r.top + lane] = wt;
   }
 }
 
-// Few pairs (T * top <= 1024, E <= 256; decoding): the choice, the counts and the places in ONE workgroup -- the same ids, weights
-// and row order as the three launches below.
-template <int SCORING>
-__global__ __launch_bounds__(256) void moe_route_small_kernel(const float* __restrict__ logits, long ldl, const void* __restrict__ corr, int cdt,
-                                                              int32_t* __restrict__ ids, float* __restrict__ wts, int32_t* __restrict__ counts,
-                                                              int32_t* __restrict__ seg, int32_t* __restrict__ src_row, int32_t* __restrict__ dst,
-                                                              int T, int E, int top, int ngroups, int keep) {
+// Few rows (T <= 64, T * top <= 1024, E <= 256; decoding): the choice, the counts and the places in ONE workgroup -- the same ids,
+// weights and row order as the three launches below.
+template <int SCORING, int NE>
+__global__ __launch_bounds__(1024) void moe_route_small_kernel(const float* __restrict__ logits, long ldl, RouteRule r, int32_t* __restrict__ ids,
+                                                               float* __restrict__ wts, int32_t* __restrict__ counts, int32_t* __restrict__ seg,
+                                                               int32_t* __restrict__ src_row, int32_t* __restrict__ dst, int T) {
+  extern __shared__ float route_vals[];
   __shared__ int ids_s[1024];
   __shared__ int cnt_s[256];
-  const int tid = threadIdx.x, R = T * top;
-  for (int t = tid; t < T; t += 256) {
-    int bi[32];
-    float w[32];
-    route_token<SCORING>(logits + (size_t)t * ldl, corr, cdt, E, top, ngroups, keep, bi, w);
-    for (int k = 0; k < top; ++k) {
-      ids[(size_t)t * top + k] = ids_s[t * top + k] = bi[k];
-      wts[(size_t)t * top + k] = w[k];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, E = r.E, top = r.top, R = T * top;
+  for (int t = wave; t < T; t += 16) {
+    int id;
+    float wt;
+    route_wave<SCORING, NE>(logits + (size_t)t * ldl, r, route_vals + (size_t)wave * E, id, wt);
+    if (lane < top) {
+      ids[(size_t)t * top + lane] = ids_s[t * top + lane] = id;
+      wts[(size_t)t * top + lane] = wt;
     }
   }
   __syncthreads();
   int c = 0;
   if (tid < E) {
-    for (int r = 0; r < R; ++r) c += ids_s[r] == tid;
+    for (int x = 0; x < R; ++x) c += ids_s[x] == tid;
     cnt_s[tid] = c;
     counts[tid] = c;
   }
@@ -116,10 +171,10 @@ __global__ __launch_bounds__(256) void moe_route_small_kernel(const float* __res
     for (int x = 0; x < tid; ++x) pos += cnt_s[x];
     seg[tid] = pos;
     if (tid == E - 1) seg[E] = pos + c;
-    for (int r = 0; r < R; ++r)
-      if (ids_s[r] == tid) {
-        src_row[pos] = r / top;
-        dst[r] = pos;
+    for (int x = 0; x < R; ++x)
+      if (ids_s[x] == tid) {
+        src_row[pos] = x / top;
+        dst[x] = pos;
         ++pos;
       }
   }
@@ -204,22 +259,32 @@ using namespace dihip;
 extern "C" {
 
 int dihip_seq_moe_route(void* stream, const float* logits, long ldl, int32_t* ids, float* wts, int32_t* counts, int32_t* seg, int32_t* src_row,
-                    int32_t* dst, int T, int E, int top, int scoring, const void* correction, int w_dtype, int ngroups, int keep) {
-  DIHIP_REQUIRE(ngroups >= 1 && ngroups <= 32 && E % ngroups == 0 && keep >= 1 && keep <= ngroups && (long)keep * (E / ngroups) >= top,
-                DIHIP_PARAM_ERROR, "moe_route: at most 32 equal groups, of which the kept ones must hold the choices");
-  DIHIP_REQUIRE((scoring == 0 || scoring == 1) && (!correction || scoring == 1) && seq_dtype_ok(w_dtype), DIHIP_PARAM_ERROR,
-                "moe_route: unknown scoring (a correction goes with scoring 1)");
-  DIHIP_REQUIRE(T >= 0 && E > 0 && top > 0 && top <= E && top <= 32 && E <= 65535 && logits && ids && wts && counts && seg && src_row && dst &&
-                    ldl >= E, DIHIP_PARAM_ERROR, "moe_route: bad argument (at most 32 choices per token)");
+                        int32_t* dst, int T, int E, int top, int scoring, const void* correction, int w_dtype, int ngroups, int keep,
+                        int group_top2, int renorm, float factor) {
+  DIHIP_REQUIRE(ngroups >= 1 && ngroups <= 64 && E % ngroups == 0 && keep >= 1 && keep <= ngroups && (long)keep * (E / ngroups) >= top,
+                DIHIP_PARAM_ERROR, "moe_route: at most 64 equal groups, of which the kept ones must hold the choices");
+  DIHIP_REQUIRE(scoring >= 0 && scoring <= 2 && (!correction || scoring > 0) && seq_dtype_ok(w_dtype), DIHIP_PARAM_ERROR,
+                "moe_route: unknown scoring (a correction goes with scoring 1 and 2)");
+  DIHIP_REQUIRE(T >= 0 && E > 0 && top > 0 && top <= E && top <= 32 && E <= 1024 && logits && ids && wts && counts && seg && src_row && dst &&
+                    ldl >= E, DIHIP_PARAM_ERROR, "moe_route: bad argument (at most 1024 experts, 32 choices per token)");
   if (T == 0) return DIHIP_SUCCESS;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  if ((long)T * top <= 1024 && E <= 256) {
-    if (scoring == 1) hipLaunchKernelGGL(moe_route_small_kernel<1>, dim3(1), dim3(256), 0, s, logits, ldl, correction, w_dtype, ids, wts, counts, seg, src_row, dst, T, E, top, ngroups, keep);
-    else hipLaunchKernelGGL(moe_route_small_kernel<0>, dim3(1), dim3(256), 0, s, logits, ldl, correction, w_dtype, ids, wts, counts, seg, src_row, dst, T, E, top, ngroups, keep);
-    return launch_status();
-  }
-  if (scoring == 1) hipLaunchKernelGGL(moe_route_kernel<1>, dim3((T + 255) / 256), dim3(256), 0, s, logits, ldl, correction, w_dtype, ids, wts, T, E, top, ngroups, keep);
-  else hipLaunchKernelGGL(moe_route_kernel<0>, dim3((T + 255) / 256), dim3(256), 0, s, logits, ldl, correction, w_dtype, ids, wts, T, E, top, ngroups, keep);
+  const RouteRule r{correction, w_dtype, E, top, ngroups, keep, group_top2, renorm, factor};
+  const bool small = T <= 64 && T * top <= 1024 && E <= 256;
+  auto go = [&](auto sc, auto ne) {
+    constexpr int SC = decltype(sc)::value, NE = decltype(ne)::value;
+    if (small) hipLaunchKernelGGL((moe_route_small_kernel<SC, NE>), dim3(1), dim3(1024), (size_t)16 * E * 4, s, logits, ldl, r, ids, wts, counts, seg, src_row, dst, T);
+    else hipLaunchKernelGGL((moe_route_kernel<SC, NE>), dim3((T + 3) / 4), dim3(256), (size_t)4 * E * 4, s, logits, ldl, r, ids, wts, T);
+  };
+  auto by_e = [&](auto sc) {
+    if (E <= 64) go(sc, std::integral_constant<int, 1>{});
+    else if (E <= 256) go(sc, std::integral_constant<int, 4>{});
+    else go(sc, std::integral_constant<int, 16>{});
+  };
+  if (scoring == 2) by_e(std::integral_constant<int, 2>{});
+  else if (scoring == 1) by_e(std::integral_constant<int, 1>{});
+  else by_e(std::integral_constant<int, 0>{});
+  if (small) return launch_status();
   hipLaunchKernelGGL(moe_count_kernel, dim3(E), dim3(256), 0, s, ids, T * top, counts);
   hipLaunchKernelGGL(moe_place_kernel, dim3(E), dim3(256), 0, s, ids, T * top, top, E, counts, seg, src_row, dst);
   return launch_status();

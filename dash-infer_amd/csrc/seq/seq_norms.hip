@@ -311,11 +311,12 @@ __global__ __launch_bounds__(NT) void gate_group_rmsnorm_reg_kernel(void* __rest
 }
 
 // ckv: rows [R latent | rot shared key part]; q_rot: rows [H][rot]; ql: rows [H][Rp], the absorbed queries in the first R columns
-// of every head.  Rotation of the two halves of the rot dimensions: (u, v) -> (u cos - v sin, v cos + u sin), angle = pos * freq[i].
-template <int WT>
+// of every head.  Rotation of dimension pairs (u, v) -> (u cos - v sin, v cos + u sin), angle = pos * freq[i], cos and sin times mag;
+// PAIRS: dimensions 2i and 2i + 1 form pair i, else i and i + rot / 2.
+template <int WT, bool PAIRS>
 __global__ __launch_bounds__(256) void latent_rope_append_kernel(void* const* __restrict__ spans, int span_stride, int span_len, int cdt,
                                                                  const float* __restrict__ ckv, long ldc, const void* __restrict__ gamma,
-                                                                 float eps, int R, int rot, int Rp, const float* __restrict__ freq,
+                                                                 float eps, int R, int rot, int Rp, const float* __restrict__ freq, float mag,
                                                                  const float* __restrict__ q_rot, long ldqr, float* __restrict__ ql, long ldql,
                                                                  int H, const int32_t* __restrict__ tok_slot,
                                                                  const int32_t* __restrict__ tok_pos) {
@@ -324,9 +325,17 @@ __global__ __launch_bounds__(256) void latent_rope_append_kernel(void* const* __
   const int t = blockIdx.x, half = rot >> 1;
   const int pos = tok_pos[t];
   for (int i = threadIdx.x; i < half; i += 256) {
-    rope_sincos((uint32_t)pos, freq[i], &sn[i], &cs[i]);
+    float s, c;
+    rope_sincos((uint32_t)pos, freq[i], &s, &c);
+    sn[i] = s * mag;
+    cs[i] = c * mag;
   }
   __syncthreads();
+  auto turn = [&](const float* p, int i) {      // element i of the rotated part at p
+    const int j = PAIRS ? i >> 1 : (i < half ? i : i - half);
+    const float u = PAIRS ? p[2 * j] : p[j], w = PAIRS ? p[2 * j + 1] : p[half + j];
+    return (PAIRS ? (i & 1) == 0 : i < half) ? u * cs[j] - w * sn[j] : w * cs[j] + u * sn[j];
+  };
   if (spans) {
     const float* cr = ckv + (size_t)t * ldc;
     float ss = 0.f;
@@ -338,17 +347,14 @@ __global__ __launch_bounds__(256) void latent_rope_append_kernel(void* const* __
       float v = 0.f;
       if (k < R) v = cr[k] * inv * load_ft<WT>(gamma, k);
       else if (k < R + rot) {
-        const int i = k - R, j = i < half ? i : i - half;
-        const float u = cr[R + j], w = cr[R + half + j];
-        v = i < half ? u * cs[j] - w * sn[j] : w * cs[j] + u * sn[j];
+        v = turn(cr + R, k - R);
       }
       st_any(span, base + k, cdt, v);
     }
   }
   for (int e = threadIdx.x; e < H * rot; e += 256) {
-    const int h = e / rot, i = e - h * rot, j = i < half ? i : i - half;
-    const float u = q_rot[(size_t)t * ldqr + (size_t)h * rot + j], w = q_rot[(size_t)t * ldqr + (size_t)h * rot + half + j];
-    ql[(size_t)t * ldql + (size_t)h * Rp + R + i] = i < half ? u * cs[j] - w * sn[j] : w * cs[j] + u * sn[j];
+    const int h = e / rot, i = e - h * rot;
+    ql[(size_t)t * ldql + (size_t)h * Rp + R + i] = turn(q_rot + (size_t)t * ldqr + (size_t)h * rot, i);
   }
 }
 
@@ -423,16 +429,20 @@ int dihip_gate_group_rmsnorm(void* stream, void* y, int y_dtype, long ldy, const
 }
 
 int dihip_latent_rope_append(void* stream, void* const* spans, int span_stride, int span_len, int cache_dtype, const float* ckv, long ldc,
-                             const void* gamma, int w_dtype, float eps, int R, int rot, int Rp, const float* freq, const float* q_rot, long ldqr,
-                             float* ql, long ldql, int H, const int32_t* tok_slot, const int32_t* tok_pos, int T) {
+                             const void* gamma, int w_dtype, float eps, int R, int rot, int Rp, const float* freq, int layout, float mag,
+                             const float* q_rot, long ldqr, float* ql, long ldql, int H, const int32_t* tok_slot, const int32_t* tok_pos, int T) {
   DIHIP_REQUIRE(T >= 0 && R > 0 && rot >= 0 && rot % 2 == 0 && rot <= 512 && Rp >= R + rot && H > 0 && q_rot && ql && tok_slot && tok_pos &&
-                    (rot == 0 || freq) && ldqr >= (long)H * rot && ldql >= (long)H * Rp && seq_dtype_ok(cache_dtype) && seq_dtype_ok(w_dtype),
+                    (rot == 0 || freq) && (layout == 0 || layout == 1) && ldqr >= (long)H * rot && ldql >= (long)H * Rp && seq_dtype_ok(cache_dtype) && seq_dtype_ok(w_dtype),
                 DIHIP_PARAM_ERROR, "latent_rope_append: bad argument (an even number of at most 512 rotated dimensions)");
   DIHIP_REQUIRE(!spans || (ckv && gamma && ldc >= R + rot && span_stride > 0 && span_len > 0), DIHIP_PARAM_ERROR,
                 "latent_rope_append: a cache needs the rows to append and the norm's weight");
   if (T == 0) return DIHIP_SUCCESS;
-  BY_WT(latent_rope_append_kernel, w_dtype, dim3(T), dim3(256), 0, reinterpret_cast<hipStream_t>(stream), spans, span_stride, span_len, cache_dtype,
-        ckv, ldc, gamma, eps, R, rot, Rp, freq, q_rot, ldqr, ql, ldql, H, tok_slot, tok_pos);
+  auto go = [&](auto kernel) {
+    hipLaunchKernelGGL(kernel, dim3(T), dim3(256), 0, reinterpret_cast<hipStream_t>(stream), spans, span_stride, span_len, cache_dtype, ckv, ldc, gamma,
+                       eps, R, rot, Rp, freq, mag, q_rot, ldqr, ql, ldql, H, tok_slot, tok_pos);
+  };
+  if (w_dtype == DIHIP_F32) layout == 0 ? go(latent_rope_append_kernel<DIHIP_F32, true>) : go(latent_rope_append_kernel<DIHIP_F32, false>);
+  else layout == 0 ? go(latent_rope_append_kernel<DIHIP_BF16, true>) : go(latent_rope_append_kernel<DIHIP_BF16, false>);
   return launch_status();
 }
 

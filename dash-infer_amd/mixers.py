@@ -3,8 +3,9 @@
 A mixer maps the rows h [T, width] (f32) of one step -- portions of several sequences, described by the step context --
 to rows of the same shape, reading and updating what its sequences left in the state manager:
   LatentWindowAttention  attention through a low-rank latent that alone is cached (paged), sliding window, softmax sink,
-                         sigmoid output gate; a layer may read the latent cache another layer writes; option: a rotated part of
-                         every head's query against ONE rotated key part per token, cached behind the latent
+                         sigmoid output gate (per element or per head); a layer may read the latent cache another layer writes;
+                         option: a rotated part of every head's query against ONE rotated key part per token, cached behind the
+                         latent (both rotary layouts, frequencies rescaled for longer contexts)
   GatedLinearRecurrence  two-branch recurrent block: gelu branch x (short causal convolution -> block-diagonal gates ->
                          real-gated diagonal recurrence), f32 state and convolution tail per slot
   DenseMlp               down(act(up(h))); act: an elementwise activation, or ("polynorm", coef): a cubic of row-normalised powers
@@ -21,10 +22,11 @@ to rows of the same shape, reading and updating what its sequences left in the s
   StateSpaceMixer        state-space duality form: short causal convolution + silu on [x | B | C], a scalar decay per head from a
                          softplus step size, a matrix state per head (f32, per slot), skip term, silu gate BEFORE a grouped RMS norm
   SideBySide             two mixers on the same input, their results RMS-normed over the width, weighted and averaged
-  GatedMlp               down(act(gate(h)) * up(h))
-  ExpertMlp              top-k routed experts; units: clamped sigmoid-gated or silu-gated; routing: softmax over the chosen logits,
-                         or softmax scores over all router outputs with a correction added for the choice alone; router outputs
-                         past the real experts stand for identity experts; an always-on shared expert
+  GatedMlp               down(act(gate(h)) * up(h)); or the clamped sigmoid-gated unit
+  ExpertMlp              top-k routed experts; units: clamped sigmoid-gated, silu-gated, or an elementwise activation without a gate;
+                         routing: softmax over the chosen logits, or softmax / sigmoid scores with a correction added for the choice
+                         alone (weights over their sum or as they are, times a factor), the choice limited to the best groups of
+                         experts; router outputs past the real experts stand for identity experts; an always-on shared expert
 Matrix products run in ctx.math (seq_ops.MATH_F32 / MATH_BF16); norms, scores, gates of the recurrence, decays and
 state are f32 in both.
 """
@@ -53,14 +55,15 @@ class StepContext:
 
 class LatentWindowAttention:
     def __init__(self, key, heads, dim, vdim, kv_rank, q_rank, window, scale, w, state, cache_dtype, kv_from_key=None, rot_dim=0,
-                 rot_base=10000.0):
+                 rot_base=10000.0, rot_layout="halves", rot_scaling=None, head_gate=False):
         """w: dq [q_rank, width], dq.norm, uq [heads*(dim+rot_dim), q_rank], dkv [kv_rank+rot_dim, width] + dkv.norm (absent with
-        kv_from_key), uk [heads*dim, kv_rank], uv [heads*vdim, kv_rank], sink [heads] (optional), g [heads*vdim, width],
-        o [width, heads*vdim].
+        kv_from_key), uk [heads*dim, kv_rank], uv [heads*vdim, kv_rank], sink [heads] (optional), g [heads*vdim, width]
+        (head_gate: [heads, width], one number per head), o [width, heads*vdim].
         rot_dim > 0: every head's query is [dim | rot_dim] and the last rot_dim rows of dkv are one key part shared by the heads;
-        both rotate with the position (halves layout, base rot_base) and add q_rot . k_rot to the score.  The page row is then
-        [latent | rotated key part | zeros up to a multiple of 32]: the attention kernels see a latent of that width, the
-        absorbed queries carry their rotated part behind them, and the value product's weight has zero columns there."""
+        both rotate with the position (rot_layout "halves" or "pairs", base rot_base, rot_scaling as rotary_frequencies takes it)
+        and add q_rot . k_rot to the score.  The page row is then [latent | rotated key part | zeros up to a multiple of 32]: the
+        attention kernels score against rows of that width, the absorbed queries carry their rotated part behind them, and the
+        row's first kv_rank elements (in whole 16-element steps for the matrix cores) are the value."""
         self.H, self.D, self.V, self.R, self.Q, self.window, self.scale = heads, dim, vdim, kv_rank, q_rank, int(window or 0), float(scale)
         self.rot = int(rot_dim or 0)
         assert self.rot % 2 == 0
@@ -69,7 +72,9 @@ class LatentWindowAttention:
         self.w_in = torch.cat(parts, 0).contiguous()          # one product for everything that reads h
         self.c_lo = q_rank
         self.g_lo = q_rank + (kv_rank + self.rot if self.owns_cache else 0)
-        self.n_in = self.g_lo + heads * vdim
+        self.head_gate = bool(head_gate)
+        self.n_in = self.g_lo + heads * (1 if head_gate else vdim)
+        assert w["g"].shape[0] == self.n_in - self.g_lo
         self.dq_norm = w["dq.norm"]
         self.dkv_norm = w.get("dkv.norm")
         assert w["uq"].shape == (heads * (dim + self.rot), q_rank) and w["o"].shape[1] == heads * vdim
@@ -80,7 +85,8 @@ class LatentWindowAttention:
             self.Rp = -(-(kv_rank + self.rot) // 32) * 32 if cache_dtype == torch.bfloat16 else kv_rank + self.rot
             uq = w["uq"].view(heads, dim + self.rot, q_rank)       # queries come out as [all heads' plain parts | all heads' rotated parts]
             self.uq = torch.cat([uq[:, :dim].reshape(heads * dim, q_rank), uq[:, dim:].reshape(heads * self.rot, q_rank)], 0).contiguous()
-            self.freq = rotary_frequencies(self.rot, rot_base)[0].to(dev)
+            f, self.mag = rotary_frequencies(self.rot, rot_base, rot_scaling)
+            self.freq, self.layout = f.to(dev), so.ROTARY_LAYOUTS[rot_layout]
         else:
             self.Rp, self.uq, self.freq = kv_rank, w["uq"].contiguous(), None
         pad = self.Rp - kv_rank
@@ -89,15 +95,19 @@ class LatentWindowAttention:
         uv = w["uv"].view(heads, vdim, kv_rank)                                            # [H, V, R]
         if pad:
             uk_t = torch.cat([uk_t, torch.zeros(heads, pad, dim, dtype=uk_t.dtype, device=dev)], 1)
-            uv = torch.cat([uv, torch.zeros(heads, vdim, pad, dtype=uv.dtype, device=dev)], 2)
-        self.uk_t, self.uv = uk_t.contiguous(), uv.contiguous()
+        self.uk_t = uk_t.contiguous()
         self.sink, self.o = w.get("sink"), w["o"].contiguous()
         if self.owns_cache:
             self.table = state.add_span_cache(key, self.Rp, cache_dtype)
         else:
             self.table = state.tables[kv_from_key]
             assert self.table.row_elems == self.Rp, "a shared latent cache must have this layer's rank (and rotated part)"
-        self.mc = so.latent_attn_mc_supported(self.table) and (heads * self.Rp) % 4 == 0
+        VW = -(-kv_rank // 16) * 16
+        self.mc = so.latent_attn_mc_supported(self.table) and (heads * self.Rp) % 4 == 0 and VW <= min(self.Rp, 512)
+        self.VW = VW if self.mc else kv_rank      # the row's elements the value product reads
+        if self.VW > kv_rank:
+            uv = torch.cat([uv, torch.zeros(heads, vdim, self.VW - kv_rank, dtype=uv.dtype, device=dev)], 2)
+        self.uv = uv.contiguous()
 
     def __call__(self, ctx, h, h16=None):
         """h16: the bf16 copy of h where the producer made one (bf16 products read it: the same bits at half the traffic)"""
@@ -108,7 +118,7 @@ class LatentWindowAttention:
             q = so.linear(cq, self.uq, math=ctx.math)
             ql = so.linear(q[:, : H * D], self.uk_t, groups=H, math=ctx.math)
             so.latent_rope_append(self.table, a[:, self.c_lo: self.g_lo], self.dkv_norm, ctx.eps, self.R, self.rot, self.freq, q[:, H * D:],
-                                  ql, H, ctx.tok_slot, ctx.tok_pos, append=self.owns_cache)
+                                  ql, H, ctx.tok_slot, ctx.tok_pos, append=self.owns_cache, layout=self.layout, mag=self.mag)
         else:
             q = so.linear(cq, self.uq, math=ctx.math, out=ctx.act_buffer(H * D))
             if self.owns_cache:
@@ -116,10 +126,10 @@ class LatentWindowAttention:
             ql = so.linear(q, self.uk_t, groups=H, math=ctx.math)
         if ctx.math == so.MATH_BF16 and self.mc:
             ol = so.latent_window_attn_mc(ql, self.table, self.sink, ctx.tok_pos, ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count,
-                                          ctx.max_pos, H, self.window, self.scale)
+                                          ctx.max_pos, H, self.window, self.scale, value=self.VW)
         else:
-            ol = so.latent_window_attn(ql, self.table, self.sink, ctx.tok_slot, ctx.tok_pos, H, self.window, self.scale, math=ctx.math)
-        og = so.linear(ol, self.uv, groups=H, mul=a[:, self.g_lo:], math=ctx.math, out=ctx.act_buffer(H * self.V))
+            ol = so.latent_window_attn(ql, self.table, self.sink, ctx.tok_slot, ctx.tok_pos, H, self.window, self.scale, math=ctx.math, value=self.VW)
+        og = so.linear(ol, self.uv, groups=H, mul=a[:, self.g_lo:], mul_group=self.head_gate, math=ctx.math, out=ctx.act_buffer(H * self.V))
         return so.linear(og, self.o, math=ctx.math)
 
 
@@ -192,8 +202,6 @@ def rotary_frequencies(dims, base, scaling=None):
 
 
 class GroupedQueryAttention:
-    LAYOUTS = {"pairs": 0, "halves": 1}
-
     def __init__(self, key, heads, kv_heads, dim, vdim, scale, w, state, cache_dtype, rot_dims=0, rot_base=10000.0, rot_layout="pairs",
                  rot_scaling=None, qk_norm=False, sink=None, softcap=None, head_gate=False, value_mix=None, window=0, keep_first=0,
                  differential=None, runs=1, head_temp=None, talk=None, elem_gate=False):
@@ -238,7 +246,7 @@ class GroupedQueryAttention:
             b = torch.cat(b + ([zero(self.H)] if head_gate else []) + ([zero(self.H * vdim)] if elem_gate else []), 0)
             self.b_in = torch.cat([b, zero(self.n_in - b.shape[0])], 0).contiguous()
         self.q_norm, self.k_norm = (w["q.norm"].contiguous(), w["k.norm"].contiguous()) if qk_norm else (None, None)
-        self.rot_dims, self.layout = int(rot_dims), self.LAYOUTS[rot_layout]
+        self.rot_dims, self.layout = int(rot_dims), so.ROTARY_LAYOUTS[rot_layout]
         assert self.rot_dims % 2 == 0 and self.rot_dims <= dim
         self.freq, self.mag = None, 1.0
         if self.rot_dims:
@@ -370,51 +378,71 @@ class SideBySide:
         return so.rmsnorm_pair(self.left(ctx, h, h16), self.w_left, self.right(ctx, h, h16), self.w_right, self.coef, ctx.eps)
 
 
+GLU_SLOPE = 1.702    # g * sigmoid(1.702 g): the sigmoid form of gelu
+
+
 class GatedMlp:
     def __init__(self, gate, up, down, act):
-        self.gate, self.up, self.down, self.act = gate.contiguous(), up.contiguous(), down.contiguous(), act
+        """act: the name of an elementwise activation, or ("clamped", limit): down(glu(min(gate h, limit), clamp(up h, +-limit))) with
+        glu(g, u) = g sigmoid(1.702 g) (u + 1)"""
+        self.down, self.act, self.limit = down.contiguous(), act, None
+        if isinstance(act, tuple):
+            assert act[0] == "clamped"
+            self.act, self.limit = None, float(act[1])
+            self.F, self.w_gu = gate.shape[0], torch.cat([gate, up], 0).contiguous()      # one product, [gate | up]
+        else:
+            self.gate, self.up = gate.contiguous(), up.contiguous()
 
     def __call__(self, ctx, h, h16=None):
         x = h16 if h16 is not None else h
+        if self.limit is not None:
+            gu = so.linear(x, self.w_gu, math=ctx.math)
+            g = so.moe_glu(gu, self.F, self.limit, GLU_SLOPE, ctx.act_buffer(self.F))
+            return so.linear(g, self.down, math=ctx.math)
         u = so.linear(x, self.up, math=ctx.math)
         g = so.linear(x, self.gate, act=self.act, mul=u, math=ctx.math, out=ctx.act_buffer(self.gate.shape[0]))   # act(gate h) * (up h)
         return so.linear(g, self.down, math=ctx.math)
 
 
 class ExpertMlp:
-    GLU_SLOPE = 1.702    # g * sigmoid(1.702 g): the sigmoid form of gelu
-
     def __init__(self, router, router_b, gates, ups, downs, top, limit=0.0, unit="clamped", scoring="chosen_softmax", correction=None,
-                 identity=0, shared=None, groups=None):
+                 identity=0, shared=None, groups=None, group_score="max", renorm=True, factor=1.0):
         """gates / ups [ff, width] and downs [width, ff] per expert.  unit "clamped": an expert is
-        down(glu(min(gate h, limit), clamp(up h, +-limit))); "silu": down(silu(gate h) * (up h)).
-        scoring "chosen_softmax": the `top` largest router logits, weights = softmax over them alone; "scores": scores = softmax over
-        all router outputs, the choice by score + correction [experts + identity] (None: the score alone), weights = the chosen
-        scores over their sum.  identity: the last `identity` router outputs have no tensors: such an expert returns its input.
+        down(glu(min(gate h, limit), clamp(up h, +-limit))); "silu": down(silu(gate h) * (up h)); gates None: unit names an elementwise
+        activation, down(act(up h)).
+        scoring "chosen_softmax": the `top` largest router logits, weights = softmax over them alone; "scores" / "sigmoid": scores =
+        softmax over all router outputs / the sigmoid of each, the choice by score + correction [experts + identity] (None: the score
+        alone), weights = the chosen scores, over their sum with renorm, times factor.  identity: the last `identity` router outputs have no tensors: such an expert returns its input.
         shared: a feed-forward (GatedMlp) that runs for every token and is added, or None.
         groups: None or (count, keep): the router outputs form `count` equal groups of neighbours, a group counts by its largest score
-        (logit), and only experts of the `keep` best groups can be chosen."""
+        (logit), or with group_score "top2" by the sum of its two largest choice scores, and only experts of the `keep` best groups can
+        be chosen."""
         self.groups = (int(groups[0]), int(groups[1])) if groups else (1, 1)
-        self.E, self.top, self.limit = len(gates), int(top), float(limit)
-        self.unit = {"clamped": so.UNIT_CLAMPED, "silu": so.UNIT_SILU}[unit]
-        self.scoring = {"chosen_softmax": so.ROUTE_CHOSEN_SOFTMAX, "scores": so.ROUTE_SCORES}[scoring]
+        self.E, self.top, self.limit = len(ups), int(top), float(limit)
+        self.unit = {"clamped": so.UNIT_CLAMPED, "silu": so.UNIT_SILU}[unit] if gates is not None else None
+        self.act = unit if gates is None else None
+        self.scoring = {"chosen_softmax": so.ROUTE_CHOSEN_SOFTMAX, "scores": so.ROUTE_SCORES, "sigmoid": so.ROUTE_SIGMOID}[scoring]
+        self.rule = dict(group_top2={"max": False, "top2": True}[group_score], renorm=bool(renorm), factor=float(factor))
         self.identity, self.shared = int(identity), shared
         self.router, self.router_b = router.contiguous(), router_b.contiguous() if router_b is not None else None
         self.correction = correction.contiguous() if correction is not None else None
-        self.F = gates[0].shape[0]
-        self.w_gu = torch.stack([torch.cat([g, u], 0) for g, u in zip(gates, ups)]).contiguous()    # [E, 2 ff, width]
+        self.F = ups[0].shape[0]
+        self.w_up = torch.stack([torch.cat([g, u], 0) for g, u in zip(gates, ups)] if gates is not None else list(ups)).contiguous()   # [E, 2 ff or ff, width]
         self.w_down = torch.stack(list(downs)).contiguous()                                          # [E, width, ff]
         assert self.router.shape[0] == self.E + self.identity and 0 < self.top <= self.E + self.identity
-        assert self.correction is None or (self.scoring == so.ROUTE_SCORES and self.correction.shape == (self.E + self.identity,))
+        assert self.correction is None or (self.scoring != so.ROUTE_CHOSEN_SOFTMAX and self.correction.shape == (self.E + self.identity,))
 
     def __call__(self, ctx, h, h16=None):
         x = h16 if h16 is not None else h
         T, R = ctx.T, ctx.T * self.top
         logits = so.linear(x, self.router, self.router_b, math=so.MATH_F32 if ctx.math == so.MATH_F32 else so.MATH_F32_STREAM)
-        ids, wts, seg, src_row, dst = so.moe_route(logits, self.top, self.scoring, self.correction, self.groups)
+        ids, wts, seg, src_row, dst = so.moe_route(logits, self.top, self.scoring, self.correction, self.groups, **self.rule)
         # the pairs of the identity experts sort behind those of the real ones: the expert products never see their rows
-        gu = so.linear_segmented(x, self.w_gu, seg, src_row, T, R, math=ctx.math)
-        y = so.moe_glu(gu, self.F, self.limit, self.GLU_SLOPE, ctx_rows(ctx, R, self.F), unit=self.unit)
+        if self.act is not None:
+            y = so.linear_segmented(x, self.w_up, seg, src_row, T, R, act=self.act, math=ctx.math, out=ctx_rows(ctx, R, self.F))
+        else:
+            gu = so.linear_segmented(x, self.w_up, seg, src_row, T, R, math=ctx.math)
+            y = so.moe_glu(gu, self.F, self.limit, GLU_SLOPE, ctx_rows(ctx, R, self.F), unit=self.unit)
         d = so.linear_segmented(y, self.w_down, seg, None, T, R, math=ctx.math)
         add = self.shared(ctx, h, h16) if self.shared is not None else None
         return so.moe_combine(d, dst, wts, T, self.top, ids=ids if self.identity else None, n_real=self.E, own=x, add=add)

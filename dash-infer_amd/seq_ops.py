@@ -32,10 +32,12 @@ def _rows(t):
     return t.stride(0)
 
 
-def linear(x, w, bias=None, out=None, act=None, act_cols=None, mul=None, math=MATH_F32, groups=1, x_groups=None):
+def linear(x, w, bias=None, out=None, act=None, act_cols=None, mul=None, math=MATH_F32, groups=1, x_groups=None, mul_group=False,
+           act_param=0.0):
     """y = epilogue(x . w^T + bias).  w: [N, K] (groups == 1) or [groups, N, K]; x: [T, x_groups * K] (group g reads the K
     columns from (g % x_groups) * K); y: [T, groups * N].  act on the output columns act_cols = (lo, hi) (default: all);
-    mul: f32 [T, groups * N] multiplied on the output."""
+    mul: f32 [T, groups * N] multiplied on the output, or with mul_group [T, groups]: one number for all columns of a group.
+    act "softcap": act_param * tanh(v / act_param)."""
     if w.dim() == 2:
         N, K = w.shape
     else:
@@ -46,11 +48,13 @@ def linear(x, w, bias=None, out=None, act=None, act_cols=None, mul=None, math=MA
     assert x.shape[1] == xg * K and w.is_contiguous() and (bias is None or (bias.is_contiguous() and bias.dtype == w.dtype))
     y = out if out is not None else torch.empty(T, groups * N, dtype=torch.float32, device=x.device)
     assert y.shape == (T, groups * N)
+    assert mul is None or (mul.dtype == torch.float32 and mul.shape[0] == T and mul.shape[1] >= (groups if mul_group else groups * N))
     lo, hi = (0, groups * N) if act_cols is None else act_cols
     if act is None:
         lo = hi = 0
     check(lib().dihip_linear(stream(), ptr(x), dt(x), _rows(x), K, xg, ptr(w), dt(w), ptr(bias), ptr(y), dt(y), _rows(y), N,
-                             ptr(mul), _rows(mul) if mul is not None else 0, T, N, K, groups, ACT[act], lo, hi, math), "dihip_linear")
+                             ptr(mul), _rows(mul) if mul is not None else 0, 1 if mul_group else 0, T, N, K, groups, ACT[act], lo, hi, float(act_param), math),
+          "dihip_linear")
     return y
 
 
@@ -124,14 +128,16 @@ def norm_residual_mix(x_in, m, gamma, eps, x_out, stack=None, mix_w=None, n_mix=
     return x_out
 
 
-def latent_window_attn(q, table, sink, tok_slot, tok_pos, H, window, scale, math=MATH_F32, out=None):
+def latent_window_attn(q, table, sink, tok_slot, tok_pos, H, window, scale, math=MATH_F32, out=None, value=None):
+    """value: the cached row's first `value` elements are the value (default: the whole row) -> f32 [T, H * value]"""
     T = q.shape[0]
     R = table.row_elems
+    RV = R if value is None else value
     assert q.shape[1] == H * R and q.dtype == torch.float32
-    o = out if out is not None else torch.empty(T, H * R, dtype=torch.float32, device=q.device)
+    o = out if out is not None else torch.empty(T, H * RV, dtype=torch.float32, device=q.device)
     check(lib().dihip_latent_window_attn(stream(), ptr(o), _rows(o), ptr(q), _rows(q), ptr(table.ptrs), table.max_spans, table.span_len,
                                          _DT[table.dtype], ptr(sink), dt(sink) if sink is not None else 0, ptr(tok_slot), ptr(tok_pos),
-                                         T, H, R, int(window), float(scale), math), "dihip_latent_window_attn")
+                                         T, H, R, int(RV), int(window), float(scale), math), "dihip_latent_window_attn")
     return o
 
 
@@ -139,21 +145,23 @@ def latent_attn_mc_supported(table):
     return bool(lib().dihip_latent_window_attn_mc_supported(table.row_elems, table.span_len, _DT[table.dtype]))
 
 
-def latent_window_attn_mc(q, table, sink, tok_pos, ent_slot, ent_row0, ent_count, max_count, max_pos, H, window, scale, out=None, nsplit=None):
+def latent_window_attn_mc(q, table, sink, tok_pos, ent_slot, ent_row0, ent_count, max_count, max_pos, H, window, scale, out=None, nsplit=None,
+                          value=None):
     """the matrix-core form (bf16 cache): rows as portions; max_count / max_pos: the largest portion and position of the step
     (host numbers: they size the grid and the split of the key walk)"""
     T, R, E = q.shape[0], table.row_elems, ent_slot.shape[0]
-    o = out if out is not None else torch.empty(T, H * R, dtype=torch.float32, device=q.device)
+    RV = R if value is None else value
+    o = out if out is not None else torch.empty(T, H * RV, dtype=torch.float32, device=q.device)
     if nsplit is None:       # fill the chip: ~2 workgroups per CU; at least 2 key tiles (64 keys) per workgroup
         blocks = max(1, E * ((max_count * H + 63) // 64))
         keys = min(max_pos + 1, window) if window > 0 else max_pos + 1
         nsplit = max(1, min(512 // blocks, (keys + 63) // 64))
     ws = None
     if nsplit > 1:
-        ws = torch.empty(int(lib().dihip_latent_window_attn_mc_workspace_bytes(T, H, R, nsplit)), dtype=torch.uint8, device=q.device)
+        ws = torch.empty(int(lib().dihip_latent_window_attn_mc_workspace_bytes(T, H, RV, nsplit)), dtype=torch.uint8, device=q.device)
     check(lib().dihip_latent_window_attn_mc(stream(), ptr(o), _rows(o), ptr(q), _rows(q), ptr(table.ptrs), table.max_spans, table.span_len,
                                             ptr(sink), dt(sink) if sink is not None else 0, ptr(tok_pos), ptr(ent_slot), ptr(ent_row0),
-                                            ptr(ent_count), E, int(max_count), T, H, R, int(window), float(scale), int(nsplit), ptr(ws),
+                                            ptr(ent_count), E, int(max_count), T, H, R, int(RV), int(window), float(scale), int(nsplit), ptr(ws),
                                             ws.numel() if ws is not None else 0), "dihip_latent_window_attn_mc")
     return o
 
@@ -240,6 +248,7 @@ def qkv_prep_append(a, q_off, k_off, v_off, H, G, D, DV, qnorm, knorm, eps, freq
           "dihip_qkv_prep_append")
 
 
+ROTARY_LAYOUTS = {"pairs": 0, "halves": 1}      # dimension 2i turns with 2i + 1 / dimension i with i + half
 SINK_NONE, SINK_PER_HEAD, SINK_ZERO = 0, 1, 2
 
 
@@ -321,12 +330,15 @@ def head_rmsnorm_mul(x, gamma, eps, H, DV, mul=None, out=None):
     return y
 
 
-ROUTE_CHOSEN_SOFTMAX, ROUTE_SCORES = 0, 1      # weights = softmax over the chosen logits / the chosen softmax scores over their sum
+# scores: the logits (weights = softmax over the chosen ones) / softmax over all logits / the sigmoid of each logit
+ROUTE_CHOSEN_SOFTMAX, ROUTE_SCORES, ROUTE_SIGMOID = 0, 1, 2
 UNIT_CLAMPED, UNIT_SILU = 0, 1
 
 
-def moe_route(logits, top, scoring=ROUTE_CHOSEN_SOFTMAX, correction=None, groups=(1, 1)):
-    """groups = (count, keep): only experts of the `keep` best of `count` equal groups of neighbours can be chosen
+def moe_route(logits, top, scoring=ROUTE_CHOSEN_SOFTMAX, correction=None, groups=(1, 1), group_top2=False, renorm=True, factor=1.0):
+    """groups = (count, keep): only experts of the `keep` best of `count` equal groups of neighbours can be chosen; a group counts by its
+    largest score, or with group_top2 by the sum of its two largest choice scores (score + correction).  renorm: the chosen scores are
+    divided by their sum (not with ROUTE_CHOSEN_SOFTMAX, whose weights are a softmax); factor multiplies them
     -> ids [T, top] i32, wts [T, top] f32, seg [E + 1], src_row [T * top], dst [T * top]"""
     T, E = logits.shape
     dev = logits.device
@@ -337,7 +349,7 @@ def moe_route(logits, top, scoring=ROUTE_CHOSEN_SOFTMAX, correction=None, groups
     assert correction is None or (correction.shape == (E,) and correction.is_contiguous())
     check(lib().dihip_seq_moe_route(stream(), ptr(logits), _rows(logits), ptr(ids), ptr(wts), ptr(counts), ptr(seg), ptr(src_row), ptr(dst),
                                     T, E, int(top), int(scoring), ptr(correction), dt(correction) if correction is not None else F32_CODE,
-                                    int(groups[0]), int(groups[1])), "dihip_seq_moe_route")
+                                    int(groups[0]), int(groups[1]), 1 if group_top2 else 0, 1 if renorm else 0, float(factor)), "dihip_seq_moe_route")
     return ids.view(T, top), wts, seg, src_row, dst
 
 
@@ -402,16 +414,16 @@ def gate_group_rmsnorm(o, z, w, eps, heads, P, groups, x=None, skip=None, out=No
     return y
 
 
-def latent_rope_append(table, ckv, gamma, eps, R, rot, freq, q_rot, ql, H, tok_slot, tok_pos, append=True):
+def latent_rope_append(table, ckv, gamma, eps, R, rot, freq, q_rot, ql, H, tok_slot, tok_pos, append=True, layout=1, mag=1.0):
     """table: the SpanTable of rows [R latent | rot key part | padding]; append False: only the queries' rotated parts are written
-    (a layer that reads another layer's pages)"""
+    (a layer that reads another layer's pages); layout 0: dimension 2i turns with 2i + 1, 1: i with i + rot / 2; mag: on cos and sin"""
     T, Rp = ql.shape[0], table.row_elems
     assert ql.dtype == q_rot.dtype == torch.float32 and ql.shape[1] == H * Rp and q_rot.shape[1] == H * rot
     assert not append or (ckv.dtype == torch.float32 and ckv.shape[1] == R + rot)
     check(lib().dihip_latent_rope_append(stream(), ptr(table.ptrs) if append else None, table.max_spans, table.span_len, _DT[table.dtype],
                                          ptr(ckv) if append else None, _rows(ckv) if append else 0, ptr(gamma) if append else None,
                                          dt(gamma) if append and gamma is not None else F32_CODE, float(eps), int(R), int(rot), int(Rp),
-                                         ptr(freq), ptr(q_rot), _rows(q_rot), ptr(ql), _rows(ql), int(H), ptr(tok_slot), ptr(tok_pos), T),
+                                         ptr(freq), int(layout), float(mag), ptr(q_rot), _rows(q_rot), ptr(ql), _rows(ql), int(H), ptr(tok_slot), ptr(tok_pos), T),
           "dihip_latent_rope_append")
 
 

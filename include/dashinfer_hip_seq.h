@@ -34,11 +34,14 @@ enum { DIHIP_MATH_F32 = 0, DIHIP_MATH_BF16 = 1, DIHIP_MATH_F32_STREAM = 2 };
 /* y[g][t, n] = epilogue( sum_k x[g % x_groups][t, k] * w[g][n, k] + bias[g][n] ),  g < groups, t < T, n < N
  *   x: [T, .] rows of stride ldx, group g starts at column (g % x_groups) * x_gstride;  w: [groups][N][K] row-major,
  *   bias: [groups][N] or NULL (w_dtype);  y: rows of stride ldy, group g at column g * y_gstride;
- *   epilogue: activation `act` on the columns act_lo <= g * N + n < act_hi, then * mul[t, g * y_gstride + n] (rows of
- *   stride ldm, f32; NULL: none). */
+ *   epilogue: activation `act` (DIHIP_ACT_*, or DIHIP_SEQ_ACT_SOFTCAP: act_param * tanh(v / act_param)) on the columns
+ *   act_lo <= g * N + n < act_hi, then * mul[t, g * y_gstride + n] (rows of stride ldm, f32; NULL: none) or, with mul_group,
+ *   * mul[t, g]: one number for all of a group's columns (a gate per head). */
+enum { DIHIP_SEQ_ACT_SOFTCAP = 7 };
 int dihip_linear(void* stream, const void* x, int x_dtype, long ldx, long x_gstride, int x_groups,
                  const void* w, int w_dtype, const void* bias, void* y, int y_dtype, long ldy, long y_gstride,
-                 const float* mul, long ldm, int T, int N, int K, int groups, int act, int act_lo, int act_hi, int math);
+                 const float* mul, long ldm, int mul_group, int T, int N, int K, int groups, int act, int act_lo, int act_hi,
+                 float act_param, int math);
 
 /* The same product for rows that are grouped by owner (mixture of experts): group g owns the output rows seg[g] .. seg[g + 1]
  * (seg: [groups + 1] on the device, ascending, seg[groups] <= R), output row r reads the x row row_map[r] (NULL: r itself) and
@@ -79,10 +82,11 @@ int dihip_gate_group_rmsnorm(void* stream, void* y, int y_dtype, long ldy, const
 /* Attention through a latent with ONE rotated key part shared by the heads.  ckv[t] = [R latent | rot key part] (f32): the page
  * row of the token (Rp elements) becomes [latent / rms * gamma | rotated key part | zeros]  (spans NULL: nothing is appended --
  * a layer that reads another layer's pages).  q_rot[t] = [H][rot]: every head's rotated query part goes to ql[t][h * Rp + R ..]
- * (behind the head's absorbed query).  Rotation: dimension i with i + rot / 2 by the angle float(pos) * freq[i]. */
+ * (behind the head's absorbed query).  Rotation: dimension 2i with 2i + 1 (layout 0) or i with i + rot / 2 (layout 1) by the
+ * angle float(pos) * freq[i], cos and sin times `mag`. */
 int dihip_latent_rope_append(void* stream, void* const* spans, int span_stride, int span_len, int cache_dtype, const float* ckv,
                              long ldc, const void* gamma, int w_dtype, float eps, int R, int rot, int Rp, const float* freq,
-                             const float* q_rot, long ldqr, float* ql, long ldql, int H, const int32_t* tok_slot,
+                             int layout, float mag, const float* q_rot, long ldqr, float* ql, long ldql, int H, const int32_t* tok_slot,
                              const int32_t* tok_pos, int T);
 
 /* State-space mixer with a scalar decay per head and a matrix state [D, DV] per head and slot (the state kernels of dihip_gla):
@@ -177,15 +181,16 @@ int dihip_gla(void* stream, float* out, long ldo, const float* q, long ldq, cons
 int dihip_head_rmsnorm_mul(void* stream, void* y, int y_dtype, long ldy, const float* x, long ldx, const void* gamma,
                            int w_dtype, float eps, const float* mul, long ldm, int T, int H, int DV);
 
-/* Mixture of experts: per token the `top` experts of largest logit (ties: the lower index) and the softmax over the chosen
- * logits (scoring 0), or scores = softmax over all E logits, the `top` experts of largest score + correction[e] (correction
- * [E] of w_dtype, NULL: none) and weights = their scores / (the sum of their scores + 1e-20) (scoring 1) -> ids / wts [T, top]; the T * top (token, choice) pairs grouped by expert -> seg [E + 1], src_row [T * top] (the
- * token a sorted row reads), dst [T * top] (the sorted row of pair t * top + k); counts: [E] scratch.
- * ngroups > 1: the experts form ngroups equal groups of neighbours; a group counts by its largest score (scoring 1) or logit, and
- * only experts of the `keep` best groups can be chosen (ngroups = keep = 1: no limit). */
+/* Mixture of experts, per token: scores s = the E logits (scoring 0), softmax over them (1) or the sigmoid of each (2); the `top`
+ * experts of largest choice score s + correction[e] are chosen (ties: the lower index; correction [E] of w_dtype, NULL: none; not
+ * with scoring 0); weights = softmax over the chosen logits alone (scoring 0), else the chosen s -- over (their sum + 1e-20) with
+ * renorm -- times factor -> ids / wts [T, top]; the T * top (token, choice) pairs grouped by expert -> seg [E + 1], src_row [T * top]
+ * (the token a sorted row reads), dst [T * top] (the sorted row of pair t * top + k); counts: [E] scratch.
+ * ngroups > 1: the experts form ngroups equal groups of neighbours and only experts of the `keep` best groups can be chosen; a
+ * group counts by its largest s, or with group_top2 by the sum of its two largest choice scores (ngroups = keep = 1: no limit). */
 int dihip_seq_moe_route(void* stream, const float* logits, long ldl, int32_t* ids, float* wts, int32_t* counts, int32_t* seg,
-                    int32_t* src_row, int32_t* dst, int T, int E, int top, int scoring, const void* correction, int w_dtype,
-                    int ngroups, int keep);
+                        int32_t* src_row, int32_t* dst, int T, int E, int top, int scoring, const void* correction, int w_dtype,
+                        int ngroups, int keep, int group_top2, int renorm, float factor);
 /* unit 0: y[r, c] = g * sigmoid(slope * g) * (u + 1),  g = min(gu[r, c], limit),  u = clamp(gu[r, F + c], -limit, limit)
  * unit 1: y[r, c] = silu(gu[r, c]) * gu[r, F + c] */
 int dihip_seq_moe_glu(void* stream, void* y, int y_dtype, long ldy, const float* gu, long ldgu, int R, int F, float limit,
@@ -236,24 +241,24 @@ int dihip_norm_residual_mix(void* stream, float* x_out, const float* x_in, const
 /* Windowed attention of every row over its sequence's cached latent rows, all heads sharing the cache:
  *   s_j = scale * q[t, h, :] . c_j   for  0 <= tok_pos[t] - j < window  (window <= 0: every j <= tok_pos[t]),
  *   p = softmax over {s_j} and one extra logit sink[h] that has no value (sink NULL: none),
- *   out[t, h, :] = sum_j p_j c_j.
- * q, out: f32 [T, H, R] (rows of stride ldq / ldo); the cache holds rows of R elements of cache_dtype. */
+ *   out[t, h, :] = sum_j p_j c_j[:RV]   (the row's first RV <= R elements are the value).
+ * q [T, H, R], out [T, H, RV]: f32 (rows of stride ldq / ldo); the cache holds rows of R elements of cache_dtype. */
 int dihip_latent_window_attn(void* stream, float* out, long ldo, const float* q, long ldq, void* const* spans,
                              int span_stride, int span_len, int cache_dtype, const void* sink, int w_dtype,
-                             const int32_t* tok_slot, const int32_t* tok_pos, int T, int H, int R, int window,
+                             const int32_t* tok_slot, const int32_t* tok_pos, int T, int H, int R, int RV, int window,
                              float scale, int math);
 
-/* The same attention on the matrix cores for a bf16 cache (R a multiple of 32 up to 512, span_len a multiple of 32; see
+/* The same attention on the matrix cores for a bf16 cache (R a multiple of 32 up to 640, RV a multiple of 16 up to 512, span_len a multiple of 32; see
  * .._supported): the rows are given as portions (ent_*: [E], rows ent_row0 .. + ent_count of one slot at consecutive
  * positions from tok_pos[ent_row0]; max_count = the largest ent_count).  nsplit > 1 splits every row's key walk over
  * that many workgroups (few rows: decoding) and merges the partial softmax records in a second launch through `ws`
  * (.._workspace_bytes).  Operands are rounded to bf16, sums are f32; a row's result depends on the tiling only by rounding. */
 int dihip_latent_window_attn_mc_supported(int R, int span_len, int cache_dtype);
-size_t dihip_latent_window_attn_mc_workspace_bytes(int T, int H, int R, int nsplit);
+size_t dihip_latent_window_attn_mc_workspace_bytes(int T, int H, int RV, int nsplit);
 int dihip_latent_window_attn_mc(void* stream, float* out, long ldo, const float* q, long ldq, void* const* spans,
                                 int span_stride, int span_len, const void* sink, int w_dtype, const int32_t* tok_pos,
                                 const int32_t* ent_slot, const int32_t* ent_row0, const int32_t* ent_count, int E,
-                                int max_count, int T, int H, int R, int window, float scale, int nsplit, void* ws,
+                                int max_count, int T, int H, int R, int RV, int window, float scale, int nsplit, void* ws,
                                 size_t ws_bytes);
 
 /* u[t, c] = bias[c] + sum_{k < taps} w[c, k] * src(t, k),  src = x[t - (taps - 1 - k), c] inside the portion, else the

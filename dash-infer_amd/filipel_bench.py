@@ -75,7 +75,7 @@ def random_model(size, device="cuda", seed=0, pattern=PATTERN):
             t[p + "mlp.act"] = torch.tensor([0.7, 0.3, 0.2, 0.05], dtype=torch.bfloat16, device=device)
         elif ff == "moe":
             E, F = s["experts"], s["expert_ff"]
-            layer["mlp"] = {"kind": "moe", "expert": {"ff": F}, "router": {"experts": E, "top": s["top"], "groups": {"count": 4, "keep": 2}}}
+            layer["mlp"] = {"kind": "moe", "expert": {"ff": F}, "router": {"experts": E, "top": s["top"], "groups": {"count": s.get("groups", 4), "keep": s.get("keep", 2)}}}
             for e in range(E):
                 t[p + f"mlp.e{e}.gate"], t[p + f"mlp.e{e}.up"], t[p + f"mlp.e{e}.down"] = r(F, W), r(F, W), r(W, F)
             t[p + "mlp.router"] = r(E, W)

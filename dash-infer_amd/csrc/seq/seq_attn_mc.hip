@@ -1,14 +1,17 @@
 // seq_attn_mc.hip -- windowed sink-softmax attention over the paged latent cache on the matrix cores (bf16 cache).
 //
-// All heads of a sequence share the cached latent rows C [keys, R]: they are keys AND (their first RV elements) values.  A workgroup owns 64
-// consecutive (row, head) pairs of one portion -- 16 per wave -- and walks the key tiles of 32 cached rows its pairs can
-// see.  Per tile: S^T = C . Q^T (A = the tile's rows as they lie in LDS, B = the wave's query fragments, held in registers
-// for the whole walk), mask + running softmax on the accumulator lanes (a pair's 32 scores sit in the four 16-lane groups
-// of one lane column: permlane swaps reduce them), then O^T += C^T . P^T with P taken straight from those lanes and
-// C^T read from the same LDS tile through the transposing LDS read.  The next tile's rows are in flight meanwhile.
+// All heads of a sequence share the cached latent rows C [keys, R]: they are keys AND (their first RV elements) values.  A workgroup
+// owns 64 or 128 consecutive (row, head) pairs of one portion -- one or two tiles of 16 per wave -- and walks the key tiles of 32
+// cached rows its pairs can see.  Per tile: S^T = C . Q^T (A = the tile's rows as they lie in LDS, B = the wave's query fragments,
+// held in registers for the whole walk), mask + running softmax on the accumulator lanes (a pair's 32 scores sit in the four 16-lane
+// groups of one lane column: permlane swaps reduce them), then O^T += C^T . P^T with P taken straight from those lanes and C^T read
+// from the same LDS tile through the transposing LDS read.  The next tile's rows are in flight meanwhile (registers, then the other
+// of two LDS tiles: one barrier per tile).
+// The loops over the row are fully unrolled for the row's size class (a multiple of 64; no run-time condition inside, which would
+// put a wait behind every LDS read): the columns between R and the class hold some finite cached values against zero query elements.
 // The key walk can be split over gridDim.z workgroups (few rows: decoding); the partial (maximum, denominator, sums)
 // records are merged by a second launch.  The sink joins split 0 as the running softmax's start (maximum = sink,
-// denominator = 1).
+// denominator = 1).  A pair's own instructions and their order do not depend on how many tiles its wave owns.
 #include "seq_common.h"
 
 namespace dihip {
@@ -28,155 +31,171 @@ __device__ __forceinline__ f32x4_t mfma_bf16x(const u32x4_t& a, const u32x4_t& b
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
-template <int RMAX, int RVMAX>
+template <int RM, int VM, int QT>
 __global__ __launch_bounds__(256) void latent_attn_mc_kernel(McArgs a) {
-  constexpr int KS = RMAX / 32, DT = RVMAX / 16, UN = RMAX / 64;
-  constexpr bool PREFETCH = RMAX <= 256;  // the widest rows leave no registers for a tile in flight
+  constexpr int KS = RM / 32, DT = VM / 16, UN = RM / 64, UPR = RM / 8;   // k steps, value tiles, 16-byte units per thread and per tile row
+  constexpr int PB = RM * 2 + 16, TILE = 32 * PB;                         // bytes of an LDS row (padded: conflict-free fragments) and tile
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+  __shared__ const char* tabs[128];
   const int e = blockIdx.y, split = blockIdx.z, nsplit = gridDim.z;
   const int H = a.H, R = a.R, RV = a.RV;
   const int cnt = a.ent_count[e], row0 = a.ent_row0[e];
-  const int nrows = cnt * H, r0 = blockIdx.x * 64;
+  const int nrows = cnt * H, r0 = (gridDim.x - 1 - blockIdx.x) * (64 * QT);      // the longest walks start first
   if (r0 >= nrows) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, ni = lane & 15, kb = lane >> 4;
-  const int pitch = R + 8, pitchb = pitch * 2;
   const int pos0 = a.tok_pos[row0];
-  const int myrow = r0 + wave * 16 + ni;
-  const bool row_ok = myrow < nrows;
-  const int rr = row_ok ? myrow : nrows - 1;
-  const int tq = rr / H, h = rr - tq * H, p = pos0 + tq;
-  const int p_lo = pos0 + r0 / H, p_hi = pos0 + min(r0 + 63, nrows - 1) / H;
+  const int p_lo = pos0 + r0 / H, p_hi = pos0 + min(r0 + 64 * QT - 1, nrows - 1) / H;
   const int k_begin = a.window > 0 ? max(0, p_lo - a.window + 1) : 0;
   const int tile_lo = k_begin >> 5, tile_hi = p_hi >> 5;
   const int per = (tile_hi - tile_lo + nsplit) / nsplit;
   const int my_lo = tile_lo + split * per, my_hi = min(tile_hi, my_lo + per - 1);
 
-  u32x4_t qf[KS];
-  {
-    const float* qrow = a.q + (size_t)(row0 + tq) * a.ldq + (size_t)h * R;
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      qf[ks] = u32x4_t{0u, 0u, 0u, 0u};
-      if (ks * 32 < R) {
-        const f32x4_t lo = *reinterpret_cast<const f32x4_t*>(qrow + ks * 32 + kb * 8);
-        const f32x4_t hi = *reinterpret_cast<const f32x4_t*>(qrow + ks * 32 + kb * 8 + 4);
-        qf[ks] = u32x4_t{pack_bf16x2(lo[0], lo[1]), pack_bf16x2(lo[2], lo[3]), pack_bf16x2(hi[0], hi[1]), pack_bf16x2(hi[2], hi[3])};
-      }
-    }
-  }
-  const bool with_sink = a.sink != nullptr && split == 0;
-  float m = with_sink ? ld_any(a.sink, h, a.wdt) : -1e30f;
-  float l = with_sink ? 1.f : 0.f;
-  const f32x4_t z4 = {0.f, 0.f, 0.f, 0.f};
-  f32x4_t oacc[DT];
-#pragma unroll
-  for (int t = 0; t < DT; ++t) oacc[t] = z4;
-
   // the span pointers of the walk, staged once: a tile's loads then depend on nothing that is still in flight
-  __shared__ const char* tabs[128];
   void* const* gtab = a.spans + (size_t)a.ent_slot[e] * a.span_stride;
   const int span_lo = (my_lo * 32) / a.span_len;
   for (int i = tid; i < 128; i += 256) {
     const int sp = span_lo + i;
     tabs[i] = (sp * a.span_len <= p_hi) ? (const char*)gtab[sp] : nullptr;
   }
-  __syncthreads();
-  // a thread's 16-byte units of a tile: (key inside the tile, column) fixed for the whole walk -- the divisions are done once.
-  // A tile of 32 keys lies inside one span (span_len % 32 == 0): its span and offset are wave-uniform.
-  const int upr = R >> 3;  // 16-byte units per cached row
+  int p[QT], h[QT], tq[QT];
+  bool row_ok[QT];
+  u32x4_t qf[QT][KS];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const int myrow = r0 + (wave * QT + t) * 16 + ni;
+    row_ok[t] = myrow < nrows;
+    const int rr = row_ok[t] ? myrow : nrows - 1;
+    tq[t] = rr / H;
+    h[t] = rr - tq[t] * H;
+    p[t] = pos0 + tq[t];
+    const float* qrow = a.q + (size_t)(row0 + tq[t]) * a.ldq + (size_t)h[t] * R + kb * 8;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const bool in = ks < KS - 1 || ks * 32 < R;      // (R is a multiple of 32: only the class's last step can lie past it)
+      const float* src = qrow + (in ? ks * 32 : 0);
+      const f32x4_t lo = *reinterpret_cast<const f32x4_t*>(src), hi = *reinterpret_cast<const f32x4_t*>(src + 4);
+      qf[t][ks] = u32x4_t{pack_bf16x2(lo[0], lo[1]), pack_bf16x2(lo[2], lo[3]), pack_bf16x2(hi[0], hi[1]), pack_bf16x2(hi[2], hi[3])};
+      if (ks == KS - 1 && !in) qf[t][ks] = u32x4_t{0u, 0u, 0u, 0u};
+    }
+  }
+  const f32x4_t z4 = {0.f, 0.f, 0.f, 0.f};
+  float m[QT], l[QT];
+  f32x4_t oacc[QT][DT];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const bool with_sink = a.sink != nullptr && split == 0;
+    m[t] = with_sink ? ld_any(a.sink, h[t], a.wdt) : -1e30f;
+    l[t] = with_sink ? 1.f : 0.f;
+#pragma unroll
+    for (int d = 0; d < DT; ++d) oacc[t][d] = z4;
+  }
+  // a thread's 16-byte units of a tile: (key inside the tile, column) fixed for the whole walk.  A tile of 32 keys lies inside one
+  // span (span_len % 32 == 0): its span and offset are wave-uniform.
   int goff[UN], loff[UN];
 #pragma unroll
   for (int j = 0; j < UN; ++j) {
-    const int u = tid + 256 * j, kin = u / upr, c8 = u - kin * upr;
-    goff[j] = kin < 32 ? (kin * R + c8 * 8) * 2 : -1;
-    loff[j] = kin * pitchb + c8 * 16;
+    const int u = tid + 256 * j, kin = u / UPR, c = u - kin * UPR;
+    goff[j] = (kin * R + min(c, (R >> 3) - 1) * 8) * 2;
+    loff[j] = kin * PB + c * 16;
   }
+  __syncthreads();
   u32x4_t pre[UN];
   auto fetch = [&](int tile) {
     const int key0 = tile * 32, sp = key0 / a.span_len;
     const char* sb = (sp - span_lo < 128 ? tabs[sp - span_lo] : (const char*)gtab[sp]) + (size_t)(key0 - sp * a.span_len) * R * 2;
 #pragma unroll
-    for (int j = 0; j < UN; ++j) {
-      pre[j] = u32x4_t{0u, 0u, 0u, 0u};
-      if (goff[j] >= 0) pre[j] = gload<u32x4_t>(sb + goff[j]);
-    }
+    for (int j = 0; j < UN; ++j) pre[j] = gload<u32x4_t>(sb + goff[j]);
   };
-  if (PREFETCH && my_lo <= my_hi) fetch(my_lo);
+  auto stage = [&](unsigned char* buf) {
+#pragma unroll
+    for (int j = 0; j < UN; ++j) *reinterpret_cast<u32x4_t*>(buf + loff[j]) = pre[j];
+  };
+  if (my_lo <= my_hi) {
+    fetch(my_lo);
+    stage(smem);
+  }
+  __syncthreads();
   for (int tile = my_lo; tile <= my_hi; ++tile) {
-    if (!PREFETCH) fetch(tile);
+    const unsigned char* buf = smem + ((tile - my_lo) & 1) * TILE;
+    const bool more = tile < my_hi;
+    fetch(more ? tile + 1 : tile);
+    f32x4_t sacc[QT][2];
 #pragma unroll
-    for (int j = 0; j < UN; ++j)
-      if (goff[j] >= 0) *reinterpret_cast<u32x4_t*>(smem + loff[j]) = pre[j];
-    __syncthreads();
-    if (PREFETCH && tile + 1 <= my_hi) fetch(tile + 1);
-    f32x4_t sacc[2] = {z4, z4};
+    for (int t = 0; t < QT; ++t) sacc[t][0] = sacc[t][1] = z4;
+    const unsigned char* kr = buf + ni * PB + kb * 16;
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      if (ks * 32 < R) {
+    for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
-        for (int nt = 0; nt < 2; ++nt) {
-          const u32x4_t kf = *reinterpret_cast<const u32x4_t*>(smem + (nt * 16 + ni) * pitchb + (ks * 32 + kb * 8) * 2);
-          sacc[nt] = mfma_bf16x(kf, qf[ks], sacc[nt]);
+      for (int nt = 0; nt < 2; ++nt) {
+        const u32x4_t kf = *reinterpret_cast<const u32x4_t*>(kr + nt * 16 * PB + ks * 64);
+#pragma unroll
+        for (int t = 0; t < QT; ++t) sacc[t][nt] = mfma_bf16x(kf, qf[t][ks], sacc[t][nt]);
+      }
+    u32x4_t pf[QT];
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      float sv[2][4], mx = -INFINITY;
+#pragma unroll
+      for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int key = tile * 32 + nt * 16 + kb * 4 + r;
+          const bool vis = key <= p[t] && (a.window <= 0 || key > p[t] - a.window);
+          sv[nt][r] = vis ? sacc[t][nt][r] * a.scale : -INFINITY;
+          mx = fmaxf(mx, sv[nt][r]);
         }
+      mx = rows_max(mx);
+      const float mn = fmaxf(m[t], mx);
+      const float corr = __expf(m[t] - mn);
+      m[t] = mn;
+      float psum = 0.f, ev[2][4];
+#pragma unroll
+      for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          ev[nt][r] = __expf(sv[nt][r] - mn);
+          psum += ev[nt][r];
+        }
+      l[t] = l[t] * corr + rows_sum(psum);
+      pf[t] = u32x4_t{pack_bf16x2(ev[0][0], ev[0][1]), pack_bf16x2(ev[0][2], ev[0][3]), pack_bf16x2(ev[1][0], ev[1][1]),
+                      pack_bf16x2(ev[1][2], ev[1][3])};
+      if (__builtin_amdgcn_ballot_w64(corr != 1.f) != 0ull) {
+#pragma unroll
+        for (int d = 0; d < DT; ++d)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) oacc[t][d][r] *= corr;
       }
     }
-    float sv[2][4], mx = -INFINITY;
+    const unsigned char* tr0 = buf + (kb * 4 + (ni >> 2)) * PB + (ni & 3) * 8;
 #pragma unroll
-    for (int nt = 0; nt < 2; ++nt)
+    for (int d = 0; d < DT; ++d) {
+      const u32x2_t lo2 = lds_read_tr16(tr0 + d * 32);
+      const u32x2_t hi2 = lds_read_tr16(tr0 + d * 32 + 16 * PB);
+      const u32x4_t vf = {lo2[0], lo2[1], hi2[0], hi2[1]};
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int key = tile * 32 + nt * 16 + kb * 4 + r;
-        const bool vis = key <= p && (a.window <= 0 || key > p - a.window);
-        sv[nt][r] = vis ? sacc[nt][r] * a.scale : -INFINITY;
-        mx = fmaxf(mx, sv[nt][r]);
-      }
-    mx = rows_max(mx);
-    const float mn = fmaxf(m, mx);
-    const float corr = __expf(m - mn);
-    m = mn;
-    float psum = 0.f, ev[2][4];
-#pragma unroll
-    for (int nt = 0; nt < 2; ++nt)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        ev[nt][r] = __expf(sv[nt][r] - mn);
-        psum += ev[nt][r];
-      }
-    l = l * corr + rows_sum(psum);
-    const u32x4_t pf = {pack_bf16x2(ev[0][0], ev[0][1]), pack_bf16x2(ev[0][2], ev[0][3]), pack_bf16x2(ev[1][0], ev[1][1]),
-                        pack_bf16x2(ev[1][2], ev[1][3])};
-    if (__builtin_amdgcn_ballot_w64(corr != 1.f) != 0ull) {
-#pragma unroll
-      for (int t = 0; t < DT; ++t)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) oacc[t][r] *= corr;
+      for (int t = 0; t < QT; ++t) oacc[t][d] = mfma_bf16x(vf, pf[t], oacc[t][d]);
     }
-    const unsigned char* tr0 = smem + (kb * 4 + (ni >> 2)) * pitchb + (ni & 3) * 8;
-#pragma unroll
-    for (int t = 0; t < DT; ++t) {
-      if (t * 16 < RV) {
-        const u32x2_t lo2 = lds_read_tr16(tr0 + t * 32);
-        const u32x2_t hi2 = lds_read_tr16(tr0 + t * 32 + 16 * pitchb);
-        const u32x4_t vf = {lo2[0], lo2[1], hi2[0], hi2[1]};
-        oacc[t] = mfma_bf16x(vf, pf, oacc[t]);
-      }
-    }
+    if (more) stage(smem + ((tile + 1 - my_lo) & 1) * TILE);      // (its readers passed the barrier before this tile)
     __syncthreads();
   }
   asm volatile("s_nop 15\n\ts_nop 7" ::: "memory");
-  if (!row_ok) return;
-  if (nsplit == 1) {
-    const float inv = 1.f / l;
-    float* o = a.out + (size_t)(row0 + tq) * a.ldo + (size_t)h * RV + kb * 4;
 #pragma unroll
-    for (int t = 0; t < DT; ++t)
-      if (t * 16 < RV) *reinterpret_cast<f32x4_t*>(o + t * 16) = f32x4_t{oacc[t][0] * inv, oacc[t][1] * inv, oacc[t][2] * inv, oacc[t][3] * inv};
-  } else {
-    float* o = a.ws + ((size_t)split * a.rows_total + (size_t)(row0 + tq) * H + h) * (RV + 4);
+  for (int t = 0; t < QT; ++t) {
+    if (!row_ok[t]) continue;
+    if (nsplit == 1) {
+      const float inv = 1.f / l[t];
+      float* o = a.out + (size_t)(row0 + tq[t]) * a.ldo + (size_t)h[t] * RV + kb * 4;
 #pragma unroll
-    for (int t = 0; t < DT; ++t)
-      if (t * 16 < RV) *reinterpret_cast<f32x4_t*>(o + t * 16 + kb * 4) = oacc[t];
-    if (kb == 0) { o[RV] = m; o[RV + 1] = l; }
+      for (int d = 0; d < DT; ++d)
+        if (d * 16 < RV)
+          *reinterpret_cast<f32x4_t*>(o + d * 16) = f32x4_t{oacc[t][d][0] * inv, oacc[t][d][1] * inv, oacc[t][d][2] * inv, oacc[t][d][3] * inv};
+    } else {
+      float* o = a.ws + ((size_t)split * a.rows_total + (size_t)(row0 + tq[t]) * H + h[t]) * (RV + 4);
+#pragma unroll
+      for (int d = 0; d < DT; ++d)
+        if (d * 16 < RV) *reinterpret_cast<f32x4_t*>(o + d * 16 + kb * 4) = oacc[t][d];
+      if (kb == 0) { o[RV] = m[t]; o[RV + 1] = l[t]; }
+    }
   }
 }
 
@@ -252,13 +271,43 @@ int dihip_latent_window_attn_mc(void* stream, float* out, long ldo, const float*
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   McArgs a{out, ldo, q, ldq, spans, span_stride, span_len, sink, w_dtype, tok_pos, ent_slot, ent_row0, ent_count, H, R, RV, window, scale,
            (float*)ws, T * H};
-  const dim3 grid((unsigned)(((long)max_count * H + 63) / 64), E, nsplit);
-  const size_t lds = (size_t)32 * (R + 8) * 2;
-  if (R <= 64) hipLaunchKernelGGL((latent_attn_mc_kernel<64, 64>), grid, dim3(256), lds, s, a);
-  else if (R <= 128) hipLaunchKernelGGL((latent_attn_mc_kernel<128, 128>), grid, dim3(256), lds, s, a);
-  else if (R <= 256) hipLaunchKernelGGL((latent_attn_mc_kernel<256, 256>), grid, dim3(256), lds, s, a);
-  else if (R <= 512) hipLaunchKernelGGL((latent_attn_mc_kernel<512, 512>), grid, dim3(256), lds, s, a);
-  else hipLaunchKernelGGL((latent_attn_mc_kernel<640, 512>), grid, dim3(256), lds, s, a);
+  // two 16-pair tiles per wave halve the LDS traffic per pair: when the pairs fill the chip anyway
+  const long pairs = (long)max_count * H;
+  const bool two = (pairs + 127) / 128 * E * nsplit >= 256;
+  int status = DIHIP_SUCCESS;
+  auto go = [&](auto rm, auto vm) {
+    constexpr int RM = decltype(rm)::value, VM = decltype(vm)::value;
+    const size_t lds = 2 * 32 * (size_t)(RM * 2 + 16);
+    auto launch = [&](auto kern, int qt) {
+      if (lds > 64 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) {
+        status = DIHIP_RUNTIME_ERROR;
+        return;
+      }
+      hipLaunchKernelGGL(kern, dim3((unsigned)((pairs + 64 * qt - 1) / (64 * qt)), E, nsplit), dim3(256), lds, s, a);
+    };
+    if constexpr (RM <= 320) {      // (a wider row's queries and sums of two tiles do not fit the registers)
+      if (two) return launch(latent_attn_mc_kernel<RM, VM, 2>, 2);
+    }
+    launch(latent_attn_mc_kernel<RM, VM, 1>, 1);
+  };
+  auto by_v = [&](auto rm) {      // the value is the whole row, or lies within the class below (a rotated part behind it)
+    constexpr int RM = decltype(rm)::value, VLOW = RM > 64 ? (RM - 64 > 512 ? 512 : RM - 64) : 64;
+    if (RM > 512 || RV <= VLOW) go(rm, std::integral_constant<int, VLOW>{});
+    else go(rm, std::integral_constant<int, (RM > 512 ? 512 : RM)>{});
+  };
+  switch ((R + 63) / 64) {
+    case 1: by_v(std::integral_constant<int, 64>{}); break;
+    case 2: by_v(std::integral_constant<int, 128>{}); break;
+    case 3: by_v(std::integral_constant<int, 192>{}); break;
+    case 4: by_v(std::integral_constant<int, 256>{}); break;
+    case 5: by_v(std::integral_constant<int, 320>{}); break;
+    case 6: by_v(std::integral_constant<int, 384>{}); break;
+    case 7: by_v(std::integral_constant<int, 448>{}); break;
+    case 8: by_v(std::integral_constant<int, 512>{}); break;
+    case 9: by_v(std::integral_constant<int, 576>{}); break;
+    default: by_v(std::integral_constant<int, 640>{}); break;
+  }
+  DIHIP_REQUIRE(status == DIHIP_SUCCESS, DIHIP_RUNTIME_ERROR, "latent_window_attn_mc: the device refuses the workgroup's LDS size");
   if (nsplit > 1) hipLaunchKernelGGL(latent_attn_merge_kernel, dim3(T * H), dim3(256), 0, s, out, ldo, (const float*)ws, nsplit, T * H, H, RV);
   return launch_status();
 }

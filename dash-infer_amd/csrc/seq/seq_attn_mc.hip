@@ -31,8 +31,10 @@ __device__ __forceinline__ f32x4_t mfma_bf16x(const u32x4_t& a, const u32x4_t& b
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
+// (two waves per SIMD where the state of a wave fits 256 registers: the sums then live in vector registers, not accumulation
+// registers, and are scaled in place)
 template <int RM, int VM, int QT>
-__global__ __launch_bounds__(256) void latent_attn_mc_kernel(McArgs a) {
+__global__ __launch_bounds__(256, ((RM + VM) * QT <= 900 ? 2 : 1)) void latent_attn_mc_kernel(McArgs a) {
   constexpr int KS = RM / 32, DT = VM / 16, UN = RM / 64, UPR = RM / 8;   // k steps, value tiles, 16-byte units per thread and per tile row
   constexpr int PB = RM * 2 + 16, TILE = 32 * PB;                         // bytes of an LDS row (padded: conflict-free fragments) and tile
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -199,6 +201,198 @@ __global__ __launch_bounds__(256) void latent_attn_mc_kernel(McArgs a) {
   }
 }
 
+// Wide rows (RM > 320): 512 threads own 64 pairs and walk tiles of 64 keys.  The scores are split by pairs and keys -- wave w scores
+// pairs (w / 2) * 16 .. + 16 against keys (w % 2) * 32 .. + 32 -- and the value product by columns: every wave holds the sums of ALL 64
+// pairs for its value columns (tiles w, w + 8, ..), so that a value fragment read from LDS serves four products.  Maxima and weights
+// go through LDS (two barriers per tile).  The state of a wave (queries, sums, the next tile's rows) fits 256 registers: two waves per
+// SIMD.  A maximum moves only when it grows by more than GROW: the weights stay below exp(GROW) with the same relative rounding,
+// and the sums are rarely scaled.
+template <int RM, int VM>
+__global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
+  constexpr int KS = RM / 32, DT = VM / 16, DW = (DT + 7) / 8, UN = RM / 64, UPR = RM / 8;
+  constexpr int PB = RM * 2 + 16, TILE = 64 * PB;
+  constexpr float GROW = 8.f;
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];      // two tiles
+  __shared__ __attribute__((aligned(16))) unsigned char wts[2 * 64 * 64];    // weights (bf16): [key half][pair][16-lane group][8 keys]
+  __shared__ float stat[2][64];
+  __shared__ const char* tabs[64];
+  const int e = blockIdx.y, split = blockIdx.z, nsplit = gridDim.z;
+  const int H = a.H, R = a.R, RV = a.RV;
+  const int cnt = a.ent_count[e], row0 = a.ent_row0[e];
+  const int nrows = cnt * H, r0 = (gridDim.x - 1 - blockIdx.x) * 64;      // the longest walks start first
+  if (r0 >= nrows) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), ni = lane & 15, kb = lane >> 4;
+  const int qg = wave >> 1, kh = wave & 1;
+  const int pos0 = a.tok_pos[row0];
+  const int p_lo = pos0 + r0 / H, p_hi = pos0 + min(r0 + 63, nrows - 1) / H;
+  const int k_begin = a.window > 0 ? max(0, p_lo - a.window + 1) : 0;
+  const int tile_lo = k_begin >> 6, tile_hi = p_hi >> 6;
+  const int per = (tile_hi - tile_lo + nsplit) / nsplit;
+  const int my_lo = tile_lo + split * per, my_hi = min(tile_hi, my_lo + per - 1);
+
+  void* const* gtab = a.spans + (size_t)a.ent_slot[e] * a.span_stride;
+  const int span_lo = (my_lo * 64) / a.span_len;
+  if (tid < 64) {
+    const int sp = span_lo + tid;
+    tabs[tid] = (sp * a.span_len <= p_hi) ? (const char*)gtab[sp] : nullptr;
+  }
+  const int myrow = min(r0 + qg * 16 + ni, nrows - 1), tq = myrow / H, hq = myrow - tq * H, p = pos0 + tq;      // the pair this lane scores
+  u32x4_t qf[KS];
+  {
+    const float* qrow = a.q + (size_t)(row0 + tq) * a.ldq + (size_t)hq * R + kb * 8;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const bool in = ks < KS - 1 || ks * 32 < R;
+      const float* src = qrow + (in ? ks * 32 : 0);
+      const f32x4_t lo = *reinterpret_cast<const f32x4_t*>(src), hi = *reinterpret_cast<const f32x4_t*>(src + 4);
+      qf[ks] = u32x4_t{pack_bf16x2(lo[0], lo[1]), pack_bf16x2(lo[2], lo[3]), pack_bf16x2(hi[0], hi[1]), pack_bf16x2(hi[2], hi[3])};
+      if (ks == KS - 1 && !in) qf[ks] = u32x4_t{0u, 0u, 0u, 0u};
+    }
+  }
+  const f32x4_t z4 = {0.f, 0.f, 0.f, 0.f};
+  const bool with_sink = a.sink != nullptr && split == 0;
+  float mq = with_sink ? ld_any(a.sink, hq, a.wdt) : -1e30f;      // the scored pair's maximum; l: its denominator over this wave's keys
+  float l = with_sink && kh == 0 ? 1.f : 0.f;
+  float m[4];                                                      // the maxima of all pairs (lane column ni of four tiles)
+  f32x4_t oacc[4][DW];
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    const int rr = min(r0 + t * 16 + ni, nrows - 1);
+    m[t] = with_sink ? ld_any(a.sink, rr % H, a.wdt) : -1e30f;
+#pragma unroll
+    for (int d = 0; d < DW; ++d) oacc[t][d] = z4;
+  }
+  int goff[UN], loff[UN];
+#pragma unroll
+  for (int j = 0; j < UN; ++j) {
+    const int u = tid + 512 * j, kin = u / UPR, c = u - kin * UPR;
+    goff[j] = (kin * R + min(c, (R >> 3) - 1) * 8) * 2;
+    loff[j] = kin * PB + c * 16;
+  }
+  __syncthreads();
+  u32x4_t pre[UN];
+  auto fetch = [&](int tile) {      // a tile of 64 keys lies inside one span (span_len % 64 == 0)
+    const int key0 = tile * 64, sp = key0 / a.span_len;
+    const char* sb = (sp - span_lo < 64 ? tabs[sp - span_lo] : (const char*)gtab[sp]) + (size_t)(key0 - sp * a.span_len) * R * 2;
+#pragma unroll
+    for (int j = 0; j < UN; ++j) pre[j] = gload<u32x4_t>(sb + goff[j]);
+  };
+  auto stage = [&](unsigned char* buf) {
+#pragma unroll
+    for (int j = 0; j < UN; ++j) *reinterpret_cast<u32x4_t*>(buf + loff[j]) = pre[j];
+  };
+  if (my_lo <= my_hi) {
+    fetch(my_lo);
+    stage(smem);
+  }
+  __syncthreads();
+  for (int tile = my_lo; tile <= my_hi; ++tile) {
+    const unsigned char* buf = smem + ((tile - my_lo) & 1) * TILE;
+    fetch(min(tile + 1, my_hi));
+    f32x4_t sacc[2] = {z4, z4};
+    const unsigned char* kr = buf + (kh * 32 + ni) * PB + kb * 16;
+    constexpr int AHEAD = 8;      // fragments in flight: the scheduler would wait for every read right before its product
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+      for (int nt = 0; nt < 2; ++nt)
+        sacc[nt] = mfma_bf16x(*reinterpret_cast<const u32x4_t*>(kr + nt * 16 * PB + ks * 64), qf[ks], sacc[nt]);
+    __builtin_amdgcn_sched_group_barrier(0x100, AHEAD, 0);
+#pragma unroll
+    for (int i = 0; i < 2 * KS - AHEAD; ++i) {
+      __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
+      __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+    }
+    __builtin_amdgcn_sched_group_barrier(0x008, AHEAD, 0);
+    __builtin_amdgcn_sched_barrier(0);
+    float sv[2][4], mx = -INFINITY;
+#pragma unroll
+    for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = tile * 64 + kh * 32 + nt * 16 + kb * 4 + r;
+        const bool vis = key <= p && (a.window <= 0 || key > p - a.window);
+        sv[nt][r] = vis ? sacc[nt][r] * a.scale : -INFINITY;
+        mx = fmaxf(mx, sv[nt][r]);
+      }
+    mx = rows_max(mx);
+    if (kb == 0) stat[kh][qg * 16 + ni] = mx;
+    __syncthreads();
+    float corr[4];
+    bool grown = false;
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      const float x = fmaxf(stat[0][t * 16 + ni], stat[1][t * 16 + ni]);
+      const float mn = x > m[t] + GROW ? x : m[t];
+      corr[t] = __expf(m[t] - mn);
+      grown |= mn != m[t];
+      m[t] = mn;
+    }
+    {
+      const float x = fmaxf(stat[0][qg * 16 + ni], stat[1][qg * 16 + ni]);
+      const float mn = x > mq + GROW ? x : mq;
+      l *= __expf(mq - mn);
+      mq = mn;
+      float psum = 0.f, ev[2][4];
+#pragma unroll
+      for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          ev[nt][r] = __expf(sv[nt][r] - mn);
+          psum += ev[nt][r];
+        }
+      l += rows_sum(psum);
+      *reinterpret_cast<u32x4_t*>(wts + ((kh * 64 + qg * 16 + ni) * 4 + kb) * 16) =
+          u32x4_t{pack_bf16x2(ev[0][0], ev[0][1]), pack_bf16x2(ev[0][2], ev[0][3]), pack_bf16x2(ev[1][0], ev[1][1]), pack_bf16x2(ev[1][2], ev[1][3])};
+    }
+    if (__builtin_amdgcn_ballot_w64(grown) != 0ull) {
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int d = 0; d < DW; ++d)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) oacc[t][d][r] *= corr[t];
+    }
+    if (tile < my_hi) stage(smem + ((tile + 1 - my_lo) & 1) * TILE);      // (its readers passed the barrier above)
+    __syncthreads();
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      u32x4_t pf[4];
+#pragma unroll
+      for (int t = 0; t < 4; ++t) pf[t] = *reinterpret_cast<const u32x4_t*>(wts + ((half * 64 + t * 16 + ni) * 4 + kb) * 16);
+      const unsigned char* tr0 = buf + (half * 32 + kb * 4 + (ni >> 2)) * PB + (ni & 3) * 8;
+#pragma unroll
+      for (int d = 0; d < DW; ++d) {
+        const int col = min(wave + 8 * d, DT - 1) * 32;
+        const u32x2_t lo2 = lds_read_tr16(tr0 + col), hi2 = lds_read_tr16(tr0 + col + 16 * PB);
+        const u32x4_t vf = {lo2[0], lo2[1], hi2[0], hi2[1]};
+#pragma unroll
+        for (int t = 0; t < 4; ++t) oacc[t][d] = mfma_bf16x(vf, pf[t], oacc[t][d]);
+      }
+    }
+  }
+  __syncthreads();      // the last maxima are no longer read
+  if (kb == 0) stat[kh][qg * 16 + ni] = l;
+  __syncthreads();
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    const int rr = r0 + t * 16 + ni;
+    if (rr >= nrows) continue;
+    const int row = row0 + rr / H, h = rr % H;
+    const float den = stat[0][t * 16 + ni] + stat[1][t * 16 + ni];
+    float* o = nsplit == 1 ? a.out + (size_t)row * a.ldo + (size_t)h * RV : a.ws + ((size_t)split * a.rows_total + (size_t)row * H + h) * (RV + 4);
+    const float inv = nsplit == 1 ? 1.f / den : 1.f;
+#pragma unroll
+    for (int d = 0; d < DW; ++d) {
+      const int col = (wave + 8 * d) * 16;
+      if (col < RV)
+        *reinterpret_cast<f32x4_t*>(o + col + kb * 4) = f32x4_t{oacc[t][d][0] * inv, oacc[t][d][1] * inv, oacc[t][d][2] * inv, oacc[t][d][3] * inv};
+    }
+    if (nsplit > 1 && wave == 0 && kb == 0) { o[RV] = m[t]; o[RV + 1] = den; }
+  }
+}
+
 __global__ __launch_bounds__(256) void latent_attn_merge_kernel(float* __restrict__ out, long ldo, const float* __restrict__ ws, int nsplit,
                                                                 int rows_total, int H, int RV) {
   __shared__ float wgt[1024];
@@ -278,17 +472,20 @@ int dihip_latent_window_attn_mc(void* stream, float* out, long ldo, const float*
   auto go = [&](auto rm, auto vm) {
     constexpr int RM = decltype(rm)::value, VM = decltype(vm)::value;
     const size_t lds = 2 * 32 * (size_t)(RM * 2 + 16);
-    auto launch = [&](auto kern, int qt) {
-      if (lds > 64 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) {
+    auto launch = [&](auto kern, int threads, int per_block, size_t bytes) {
+      if (bytes > 64 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes) != hipSuccess) {
         status = DIHIP_RUNTIME_ERROR;
         return;
       }
-      hipLaunchKernelGGL(kern, dim3((unsigned)((pairs + 64 * qt - 1) / (64 * qt)), E, nsplit), dim3(256), lds, s, a);
+      hipLaunchKernelGGL(kern, dim3((unsigned)((pairs + per_block - 1) / per_block), E, nsplit), dim3(threads), bytes, s, a);
     };
-    if constexpr (RM <= 320) {      // (a wider row's queries and sums of two tiles do not fit the registers)
-      if (two) return launch(latent_attn_mc_kernel<RM, VM, 2>, 2);
+    if constexpr (RM > 320 && RM <= 576) {
+      if (span_len % 64 == 0) return launch(latent_attn_wide_kernel<RM, VM>, 512, 64, 2 * lds);
     }
-    launch(latent_attn_mc_kernel<RM, VM, 1>, 1);
+    if constexpr (RM <= 320) {      // (a wider row's queries and sums of two tiles do not fit the registers)
+      if (two) return launch(latent_attn_mc_kernel<RM, VM, 2>, 256, 128, lds);
+    }
+    launch(latent_attn_mc_kernel<RM, VM, 1>, 256, 64, lds);
   };
   auto by_v = [&](auto rm) {      // the value is the whole row, or lies within the class below (a rotated part behind it)
     constexpr int RM = decltype(rm)::value, VLOW = RM > 64 ? (RM - 64 > 512 ? 512 : RM - 64) : 64;

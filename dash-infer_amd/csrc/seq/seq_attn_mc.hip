@@ -205,12 +205,19 @@ __global__ __launch_bounds__(256, ((RM + VM) * QT <= 900 ? 2 : 1)) void latent_a
 // pairs (w / 2) * 16 .. + 16 against keys (w % 2) * 32 .. + 32 -- and the value product by columns: every wave holds the sums of ALL 64
 // pairs for its value columns (tiles w, w + 8, ..), so that a value fragment read from LDS serves four products.  Maxima and weights
 // go through LDS (two barriers per tile).  The state of a wave (queries, sums, the next tile's rows) fits 256 registers: two waves per
-// SIMD.  A maximum moves only when it grows by more than GROW: the weights stay below exp(GROW) with the same relative rounding,
+// SIMD.  The rows of a tile lie unpadded in LDS, their 16-byte units permuted inside blocks of 8 or 16 (wide_swizzle): the fragment reads
+// and the transposing reads are free of bank conflicts.  A maximum moves only when it grows by more than GROW: the weights stay below exp(GROW) with the same relative rounding,
 // and the sums are rarely scaled.
+template <int RM>
+__device__ __forceinline__ int wide_swizzle(int row) {      // unit c of the row lies at unit c ^ wide_swizzle(row)
+  const int q = (row >> 1) & 7, s = q < 4 ? 2 * q : (2 * q - 3) & 7;
+  return RM % 128 == 0 ? (row & 1) << 3 | s : s;            // (a row of an odd number of 8-unit blocks moves every other row by half the banks)
+}
+
 template <int RM, int VM>
 __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
   constexpr int KS = RM / 32, DT = VM / 16, DW = (DT + 7) / 8, UN = RM / 64, UPR = RM / 8;
-  constexpr int PB = RM * 2 + 16, TILE = 64 * PB;
+  constexpr int PB = RM * 2, TILE = 64 * PB;
   constexpr float GROW = 8.f;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];      // two tiles
   __shared__ __attribute__((aligned(16))) unsigned char wts[2 * 64 * 64];    // weights (bf16): [key half][pair][16-lane group][8 keys]
@@ -267,15 +274,23 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
   for (int j = 0; j < UN; ++j) {
     const int u = tid + 512 * j, kin = u / UPR, c = u - kin * UPR;
     goff[j] = (kin * R + min(c, (R >> 3) - 1) * 8) * 2;
-    loff[j] = kin * PB + c * 16;
+    loff[j] = kin * PB + (c ^ wide_swizzle<RM>(kin)) * 16;
   }
+  // the lane's fragment reads: four k steps span 16 units, so four offsets cover every step; its transposing reads: tiles 8 apart, one
+  const int sw = wide_swizzle<RM>(ni), vrow = kb * 4 + (ni >> 2), vsw = wide_swizzle<RM>(vrow);
+  int koff[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) koff[i] = (kh * 32 + ni) * PB + ((i * 4 + kb) ^ sw) * 16;
+  const int voff = vrow * PB + ((wave * 2 + ((ni & 3) >> 1)) ^ vsw) * 16 + (ni & 1) * 8;
   __syncthreads();
   u32x4_t pre[UN];
   auto fetch = [&](int tile) {      // a tile of 64 keys lies inside one span (span_len % 64 == 0)
     const int key0 = tile * 64, sp = key0 / a.span_len;
-    const char* sb = (sp - span_lo < 64 ? tabs[sp - span_lo] : (const char*)gtab[sp]) + (size_t)(key0 - sp * a.span_len) * R * 2;
+    const uintptr_t at = (uintptr_t)(sp - span_lo < 64 ? tabs[sp - span_lo] : (const char*)gtab[sp]);
+    const uintptr_t ua = (uintptr_t)__builtin_amdgcn_readfirstlane((unsigned)(at >> 32)) << 32 | (unsigned)__builtin_amdgcn_readfirstlane((unsigned)at);
+    const char* sb = (const char*)ua + (size_t)(key0 - sp * a.span_len) * R * 2;      // wave-uniform
 #pragma unroll
-    for (int j = 0; j < UN; ++j) pre[j] = gload<u32x4_t>(sb + goff[j]);
+    for (int j = 0; j < UN; ++j) pre[j] = gload<u32x4_t>(sb + (unsigned)goff[j]);
   };
   auto stage = [&](unsigned char* buf) {
 #pragma unroll
@@ -290,14 +305,13 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
     const unsigned char* buf = smem + ((tile - my_lo) & 1) * TILE;
     fetch(min(tile + 1, my_hi));
     f32x4_t sacc[2] = {z4, z4};
-    const unsigned char* kr = buf + (kh * 32 + ni) * PB + kb * 16;
     constexpr int AHEAD = 8;      // fragments in flight: the scheduler would wait for every read right before its product
     __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
       for (int nt = 0; nt < 2; ++nt)
-        sacc[nt] = mfma_bf16x(*reinterpret_cast<const u32x4_t*>(kr + nt * 16 * PB + ks * 64), qf[ks], sacc[nt]);
+        sacc[nt] = mfma_bf16x(*reinterpret_cast<const u32x4_t*>(buf + koff[ks & 3] + nt * 16 * PB + (ks >> 2) * 256), qf[ks], sacc[nt]);
     __builtin_amdgcn_sched_group_barrier(0x100, AHEAD, 0);
 #pragma unroll
     for (int i = 0; i < 2 * KS - AHEAD; ++i) {
@@ -307,15 +321,25 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
     __builtin_amdgcn_sched_group_barrier(0x008, AHEAD, 0);
     __builtin_amdgcn_sched_barrier(0);
     float sv[2][4], mx = -INFINITY;
+    if (tile * 64 + 63 > p_lo || (a.window > 0 && tile * 64 <= p_hi - a.window)) {      // some pair does not see the whole tile
 #pragma unroll
-    for (int nt = 0; nt < 2; ++nt)
+      for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int key = tile * 64 + kh * 32 + nt * 16 + kb * 4 + r;
-        const bool vis = key <= p && (a.window <= 0 || key > p - a.window);
-        sv[nt][r] = vis ? sacc[nt][r] * a.scale : -INFINITY;
-        mx = fmaxf(mx, sv[nt][r]);
-      }
+        for (int r = 0; r < 4; ++r) {
+          const int key = tile * 64 + kh * 32 + nt * 16 + kb * 4 + r;
+          const bool vis = key <= p && (a.window <= 0 || key > p - a.window);
+          sv[nt][r] = vis ? sacc[nt][r] * a.scale : -INFINITY;
+          mx = fmaxf(mx, sv[nt][r]);
+        }
+    } else {
+#pragma unroll
+      for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          sv[nt][r] = sacc[nt][r] * a.scale;
+          mx = fmaxf(mx, sv[nt][r]);
+        }
+    }
     mx = rows_max(mx);
     if (kb == 0) stat[kh][qg * 16 + ni] = mx;
     __syncthreads();
@@ -361,11 +385,10 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
       u32x4_t pf[4];
 #pragma unroll
       for (int t = 0; t < 4; ++t) pf[t] = *reinterpret_cast<const u32x4_t*>(wts + ((half * 64 + t * 16 + ni) * 4 + kb) * 16);
-      const unsigned char* tr0 = buf + (half * 32 + kb * 4 + (ni >> 2)) * PB + (ni & 3) * 8;
 #pragma unroll
       for (int d = 0; d < DW; ++d) {
-        const int col = min(wave + 8 * d, DT - 1) * 32;
-        const u32x2_t lo2 = lds_read_tr16(tr0 + col), hi2 = lds_read_tr16(tr0 + col + 16 * PB);
+        const unsigned char* tr0 = buf + (8 * d + 7 < DT || wave + 8 * d < DT ? voff + d * 256 : voff) + half * 32 * PB;      // (past the value: any tile, not stored)
+        const u32x2_t lo2 = lds_read_tr16(tr0), hi2 = lds_read_tr16(tr0 + 16 * PB);
         const u32x4_t vf = {lo2[0], lo2[1], hi2[0], hi2[1]};
 #pragma unroll
         for (int t = 0; t < 4; ++t) oacc[t][d] = mfma_bf16x(vf, pf[t], oacc[t][d]);
@@ -480,7 +503,7 @@ int dihip_latent_window_attn_mc(void* stream, float* out, long ldo, const float*
       hipLaunchKernelGGL(kern, dim3((unsigned)((pairs + per_block - 1) / per_block), E, nsplit), dim3(threads), bytes, s, a);
     };
     if constexpr (RM > 320 && RM <= 576) {
-      if (span_len % 64 == 0) return launch(latent_attn_wide_kernel<RM, VM>, 512, 64, 2 * lds);
+      if (span_len % 64 == 0) return launch(latent_attn_wide_kernel<RM, VM>, 512, 64, 2 * 64 * (size_t)RM * 2);
     }
     if constexpr (RM <= 320) {      // (a wider row's queries and sums of two tiles do not fit the registers)
       if (two) return launch(latent_attn_mc_kernel<RM, VM, 2>, 256, 128, lds);

@@ -152,10 +152,10 @@ def latent_window_attn_mc(q, table, sink, tok_pos, ent_slot, ent_row0, ent_count
     T, R, E = q.shape[0], table.row_elems, ent_slot.shape[0]
     RV = R if value is None else value
     o = out if out is not None else torch.empty(T, H * RV, dtype=torch.float32, device=q.device)
-    if nsplit is None:       # fill the chip: ~2 workgroups per CU; at least 2 key tiles (64 keys) per workgroup
+    if nsplit is None:       # fill the chip: ~2 workgroups per CU (wide rows: one takes a CU); at least 64 keys per workgroup
         blocks = max(1, E * ((max_count * H + 63) // 64))
         keys = min(max_pos + 1, window) if window > 0 else max_pos + 1
-        nsplit = max(1, min(512 // blocks, (keys + 63) // 64))
+        nsplit = max(1, min((256 if R > 320 else 512) // blocks, (keys + 63) // 64))
     ws = None
     if nsplit > 1:
         ws = torch.empty(int(lib().dihip_latent_window_attn_mc_workspace_bytes(T, H, RV, nsplit)), dtype=torch.uint8, device=q.device)

@@ -216,7 +216,7 @@ __device__ __forceinline__ int wide_swizzle(int row) {      // unit c of the row
 
 template <int RM, int VM>
 __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
-  constexpr int KS = RM / 32, DT = VM / 16, DW = (DT + 7) / 8, UN = RM / 64, UPR = RM / 8;
+  constexpr int KS = RM / 32, DT = VM / 16, DW = (DT + 7) / 8, UN = RM / 64;
   constexpr int PB = RM * 2, TILE = 64 * PB;
   constexpr float GROW = 8.f;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];      // two tiles
@@ -269,13 +269,11 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
 #pragma unroll
     for (int d = 0; d < DW; ++d) oacc[t][d] = z4;
   }
-  int goff[UN], loff[UN];
-#pragma unroll
-  for (int j = 0; j < UN; ++j) {
-    const int u = tid + 512 * j, kin = u / UPR, c = u - kin * UPR;
-    goff[j] = (kin * R + min(c, (R >> 3) - 1) * 8) * 2;
-    loff[j] = kin * PB + (c ^ wide_swizzle<RM>(kin)) * 16;
-  }
+  // eight threads stage a row of the tile, units (tid % 8) + 8 j: one offset into the page and two into LDS (even and odd j)
+  const int srow = tid >> 3, scol = tid & 7, ssw = wide_swizzle<RM>(srow);
+  const unsigned goff = (unsigned)(srow * R * 2 + scol * 16);
+  const unsigned glast = (unsigned)(srow * R * 2 + min(scol + 8 * (UN - 1), (R >> 3) - 1) * 16);      // (R may end inside the class's last block)
+  const int loff0 = srow * PB + (scol ^ ssw) * 16, loff1 = srow * PB + ((scol + 8) ^ ssw) * 16 - 128;
   // the lane's fragment reads: four k steps span 16 units, so four offsets cover every step; its transposing reads: tiles 8 apart, one
   const int sw = wide_swizzle<RM>(ni), vrow = kb * 4 + (ni >> 2), vsw = wide_swizzle<RM>(vrow);
   int koff[4];
@@ -290,11 +288,11 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
     const uintptr_t ua = (uintptr_t)__builtin_amdgcn_readfirstlane((unsigned)(at >> 32)) << 32 | (unsigned)__builtin_amdgcn_readfirstlane((unsigned)at);
     const char* sb = (const char*)ua + (size_t)(key0 - sp * a.span_len) * R * 2;      // wave-uniform
 #pragma unroll
-    for (int j = 0; j < UN; ++j) pre[j] = gload<u32x4_t>(sb + (unsigned)goff[j]);
+    for (int j = 0; j < UN; ++j) pre[j] = gload<u32x4_t>(sb + (j < UN - 1 ? goff + j * 128u : glast));
   };
   auto stage = [&](unsigned char* buf) {
 #pragma unroll
-    for (int j = 0; j < UN; ++j) *reinterpret_cast<u32x4_t*>(buf + loff[j]) = pre[j];
+    for (int j = 0; j < UN; ++j) *reinterpret_cast<u32x4_t*>(buf + ((j & 1) ? loff1 : loff0) + j * 128) = pre[j];
   };
   if (my_lo <= my_hi) {
     fetch(my_lo);
@@ -305,21 +303,22 @@ __global__ __launch_bounds__(512) void latent_attn_wide_kernel(McArgs a) {
     const unsigned char* buf = smem + ((tile - my_lo) & 1) * TILE;
     fetch(min(tile + 1, my_hi));
     f32x4_t sacc[2] = {z4, z4};
-    constexpr int AHEAD = 8;      // fragments in flight: the scheduler would wait for every read right before its product
-    __builtin_amdgcn_sched_barrier(0);
+    // two k steps at a time, the next two steps' fragments in flight (left alone, the scheduler puts a wait behind every read)
+    u32x4_t kf[2][4];
+    auto kload = [&](int b) {
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
+      for (int i = 0; i < 4; ++i)
+        kf[b & 1][i] = *reinterpret_cast<const u32x4_t*>(buf + koff[(2 * b + (i >> 1)) & 3] + (i & 1) * 16 * PB + ((2 * b + (i >> 1)) >> 2) * 256);
+    };
+    kload(0);
 #pragma unroll
-      for (int nt = 0; nt < 2; ++nt)
-        sacc[nt] = mfma_bf16x(*reinterpret_cast<const u32x4_t*>(buf + koff[ks & 3] + nt * 16 * PB + (ks >> 2) * 256), qf[ks], sacc[nt]);
-    __builtin_amdgcn_sched_group_barrier(0x100, AHEAD, 0);
+    for (int b = 0; b < KS / 2; ++b) {
+      if (b + 1 < KS / 2) kload(b + 1);
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int i = 0; i < 2 * KS - AHEAD; ++i) {
-      __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
-      __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      for (int i = 0; i < 4; ++i) sacc[i & 1] = mfma_bf16x(kf[b & 1][i], qf[2 * b + (i >> 1)], sacc[i & 1]);
+      __builtin_amdgcn_sched_barrier(0);
     }
-    __builtin_amdgcn_sched_group_barrier(0x008, AHEAD, 0);
-    __builtin_amdgcn_sched_barrier(0);
     float sv[2][4], mx = -INFINITY;
     if (tile * 64 + 63 > p_lo || (a.window > 0 && tile * 64 <= p_hi - a.window)) {      // some pair does not see the whole tile
 #pragma unroll

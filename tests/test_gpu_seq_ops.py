@@ -252,7 +252,8 @@ def test_gated_recurrence_portions_long_decode_and_state(so):
     assert torch.equal(one.cpu(), torch.from_numpy(np.concatenate(got))) and torch.equal(whole[1], state[1])
 
 
-@pytest.mark.parametrize("R,H,window,nsplit", [(64, 3, 37, 1), (64, 1, 64, 3), (128, 5, 130, 1), (96, 2, 0, 4), (256, 4, 65, 2), (512, 2, 200, 1), (32, 7, 33, None)])
+@pytest.mark.parametrize("R,H,window,nsplit", [(64, 3, 37, 1), (64, 1, 64, 3), (128, 5, 130, 1), (96, 2, 0, 4), (256, 4, 65, 2), (512, 2, 200, 1), (32, 7, 33, None), (192, 3, 40, 2),
+                                               (320, 6, 0, 1), (352, 3, 100, 3), (384, 1, 64, None), (416, 9, 70, 1), (448, 3, 129, 2), (480, 2, 0, 5)])
 def test_latent_window_attn_on_the_matrix_cores(so, R, H, window, nsplit):
     """the same edges, page borders and far keys through the matrix-core kernel: two portions of two slots and single rows,
     with and without a split key walk, against the float64 restatement (bf16 operands: tolerance of their rounding)"""
@@ -286,6 +287,28 @@ def test_latent_window_attn_on_the_matrix_cores(so, R, H, window, nsplit):
             shifted = attn_ref(qr, rows, pos, H, window + 1, 0.5, sink.float().numpy())
             if rel_err(shifted, want) > 0.05:
                 assert rel_err(got.cpu().numpy(), shifted) > 0.03
+
+
+@pytest.mark.parametrize("R,RV,H,window,nsplit,span", [(96, 64, 3, 37, 1, 64), (160, 128, 2, 0, 2, 64), (512, 448, 5, 65, 1, 64), (576, 512, 3, 100, 1, 64),
+                                                       (576, 512, 2, 0, 4, 64), (544, 400, 70, 130, 1, 128), (576, 512, 4, 64, 2, 32), (640, 512, 2, 33, 3, 64)])
+def test_latent_attention_whose_value_is_a_part_of_the_row(so, R, RV, H, window, nsplit, span):
+    """keys of R elements whose first RV are the value, on rows of every kernel's size (and pages of 32 rows, which the kernel with tiles
+    of 64 keys does not take); every page row past the sequence's end holds large finite values that must not be seen"""
+    rng = np.random.default_rng(R + H)
+    n = 300
+    rows = torch.from_numpy(rng.normal(0, 0.3, (n, R)).astype(np.float32)).to(torch.bfloat16).float().numpy()
+    st, tab, slot = filled_cache(np.concatenate([rows, np.full((span, R), 50.0, np.float32)]), torch.bfloat16, span_len=span)
+    sink = bf(rng.normal(0, 1, H))
+    i32 = lambda a: torch.tensor(a, dtype=torch.int32).cuda()
+    for start, count in ((0, 70), (130, 170), (n - 1, 1), (63, 2)):
+        pos = list(range(start, start + count))
+        qr = torch.from_numpy(rng.normal(0, 0.6, (count, H * R)).astype(np.float32)).to(torch.bfloat16).float().numpy()
+        want = attn_ref(qr, rows, pos, H, window, 0.5, sink.float().numpy()).reshape(count, H, R)[:, :, :RV].reshape(count, H * RV)
+        got = so.latent_window_attn_mc(dev(qr), tab, sink.cuda(), i32(pos), i32([slot.index]), i32([0]), i32([count]), count, pos[-1], H, window, 0.5,
+                                       nsplit=nsplit, value=RV)
+        assert rel_err(got.cpu().numpy(), want) < 8e-3, (start, count)
+        row = so.latent_window_attn(dev(qr), tab, sink.cuda(), torch.full((count,), slot.index, dtype=torch.int32).cuda(), i32(pos), H, window, 0.5, value=RV)
+        assert rel_err(row.cpu().numpy(), want) < 2e-5, (start, count)
 
 
 def test_gated_recurrence_in_chunks_side_by_side(so):

@@ -1,5 +1,5 @@
 // seq_norms.hip -- row operators of layers that run their sublayers side by side on a layer-normed stream (everything in f32):
-//   residual_layernorm   x_out = x_in + mult * (a + b);  h = (x_out - mean) / sqrt(var + eps) * w (+ bias)  -- the residual step of
+//   residual_layernorm   x_out = x_in + mult * (a + b + routed experts' weighted rows);  h = (x_out - mean) / sqrt(var + eps) * w (+ bias)  -- the residual step of
 //                        two sublayers and the NEXT layer's input norm in one launch; with row_idx: the norm of chosen rows alone
 //   polynorm             y = c0 z / rms(z) + c1 z^2 / rms(z^2) + c2 z^3 / rms(z^3) + c3   (powers per element, rms over the row)
 //   rmsnorm_pair         y = coef * (xa / rms(xa) * wa + xb / rms(xb) * wb)   -- two branches joined on equal footing
@@ -14,9 +14,20 @@
 namespace dihip {
 namespace {
 
+// the weighted sum of a token's routed rows (k ascending: the bits of moe_combine); dst NULL: none
+struct RoutedRows {
+  const float* rows; long ld;
+  const int32_t* dst; const float* wts; int top;
+};
+__device__ __forceinline__ float routed_sum(const RoutedRows& q, size_t r, int k) {
+  float acc = 0.f;
+  for (int j = 0; j < q.top; ++j) acc = __builtin_fmaf(q.wts[r * q.top + j], q.rows[(size_t)q.dst[r * q.top + j] * q.ld + k], acc);
+  return acc;
+}
+
 template <int WT>
 __global__ __launch_bounds__(256) void residual_layernorm_kernel(float* x_out, const float* x_in, const float* __restrict__ a, long lda,
-                                                                 const float* __restrict__ b, long ldb, float mult,
+                                                                 const float* __restrict__ b, long ldb, RoutedRows q, float mult,
                                                                  const int32_t* __restrict__ row_idx, const void* __restrict__ w,
                                                                  const void* __restrict__ bias, float eps, void* __restrict__ h, int hdt,
                                                                  long ldh, int K) {
@@ -28,9 +39,10 @@ __global__ __launch_bounds__(256) void residual_layernorm_kernel(float* x_out, c
 #pragma unroll 4
   for (int k = threadIdx.x; k < K; k += 256) {
     float v = x_in[r * K + k];
-    if (a) {
-      float s = a[r * lda + k];
+    if (a || q.dst) {
+      float s = a ? a[r * lda + k] : 0.f;
       if (b) s += b[r * ldb + k];
+      if (q.dst) s += routed_sum(q, r, k);
       v = __builtin_fmaf(mult, s, v);
     }
     if (x_out) x_out[r * K + k] = v;     // (re-read below by the thread that wrote it)
@@ -153,7 +165,7 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 
 template <int WT, int NT, int EPT>
 __global__ __launch_bounds__(NT) void residual_layernorm_reg_kernel(float* x_out, const float* x_in, const float* __restrict__ a, long lda,
-                                                                    const float* __restrict__ b, long ldb, float mult,
+                                                                    const float* __restrict__ b, long ldb, RoutedRows q, float mult,
                                                                     const int32_t* __restrict__ row_idx, const void* __restrict__ w,
                                                                     const void* __restrict__ bias, float eps, void* __restrict__ h, int hdt,
                                                                     long ldh, int K) {
@@ -163,13 +175,26 @@ __global__ __launch_bounds__(NT) void residual_layernorm_reg_kernel(float* x_out
   float v[EPT];
 #pragma unroll
   for (int e = 0; e < EPT; ++e) v[e] = x_in[r * K + min(tid + e * NT, K - 1)];
-  if (a) {
+  if (a || q.dst) {
     float s[EPT];
 #pragma unroll
-    for (int e = 0; e < EPT; ++e) s[e] = a[r * lda + min(tid + e * NT, K - 1)];
+    for (int e = 0; e < EPT; ++e) s[e] = a ? a[r * lda + min(tid + e * NT, K - 1)] : 0.f;
     if (b) {
 #pragma unroll
       for (int e = 0; e < EPT; ++e) s[e] += b[r * ldb + min(tid + e * NT, K - 1)];
+    }
+    if (q.dst) {
+      float acc[EPT];
+#pragma unroll
+      for (int e = 0; e < EPT; ++e) acc[e] = 0.f;
+      for (int j = 0; j < q.top; ++j) {
+        const float wt = q.wts[r * q.top + j];
+        const float* row = q.rows + (size_t)q.dst[r * q.top + j] * q.ld;
+#pragma unroll
+        for (int e = 0; e < EPT; ++e) acc[e] = __builtin_fmaf(wt, row[min(tid + e * NT, K - 1)], acc[e]);
+      }
+#pragma unroll
+      for (int e = 0; e < EPT; ++e) s[e] += acc[e];
     }
 #pragma unroll
     for (int e = 0; e < EPT; ++e) v[e] = __builtin_fmaf(mult, s[e], v[e]);
@@ -387,14 +412,15 @@ using namespace dihip;
 
 extern "C" {
 
-int dihip_residual_layernorm(void* stream, float* x_out, const float* x_in, const float* a, long lda, const float* b, long ldb, float mult,
-                             const int32_t* row_idx, const void* w, const void* bias, int w_dtype, float eps, void* h, int h_dtype, long ldh,
+int dihip_residual_layernorm(void* stream, float* x_out, const float* x_in, const float* a, long lda, const float* b, long ldb,
+                             const float* rows, long ldr, const int32_t* dst, const float* wts, int top, float mult, const int32_t* row_idx, const void* w, const void* bias, int w_dtype, float eps, void* h, int h_dtype, long ldh,
                              int M, int K) {
   DIHIP_REQUIRE(M >= 0 && K > 0 && x_in && (!a || lda >= K) && (!b || (a && ldb >= K)) && (!w || (h && ldh >= K)) && (!row_idx || !x_out) &&
-                    (x_out || !a) && seq_dtype_ok(w_dtype) && seq_dtype_ok(h_dtype), DIHIP_PARAM_ERROR, "residual_layernorm: bad argument");
+                    (x_out || (!a && !dst)) && seq_dtype_ok(w_dtype) && seq_dtype_ok(h_dtype), DIHIP_PARAM_ERROR, "residual_layernorm: bad argument");
+  DIHIP_REQUIRE(!dst || (rows && wts && top > 0 && ldr >= K), DIHIP_PARAM_ERROR, "residual_layernorm: routed rows need their weights and places");
   if (M == 0) return DIHIP_SUCCESS;
-  BY_WT_ROW(residual_layernorm, K, w_dtype, dim3(M), reinterpret_cast<hipStream_t>(stream), x_out, x_in, a, lda, b, ldb, mult, row_idx, w, bias,
-            eps, h, h_dtype, ldh, K);
+  BY_WT_ROW(residual_layernorm, K, w_dtype, dim3(M), reinterpret_cast<hipStream_t>(stream), x_out, x_in, a, lda, b, ldb,
+            (RoutedRows{rows, ldr, dst, wts, top}), mult, row_idx, w, bias, eps, h, h_dtype, ldh, K);
   return launch_status();
 }
 

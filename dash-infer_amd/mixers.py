@@ -432,7 +432,9 @@ class ExpertMlp:
         assert self.router.shape[0] == self.E + self.identity and 0 < self.top <= self.E + self.identity
         assert self.correction is None or (self.scoring != so.ROUTE_CHOSEN_SOFTMAX and self.correction.shape == (self.E + self.identity,))
 
-    def __call__(self, ctx, h, h16=None):
+    def __call__(self, ctx, h, h16=None, defer=False):
+        """defer: where the result is nothing but the weighted sum of routed rows, (rows, dst, wts) is returned instead, to be summed
+        inside the residual step (seq_ops.residual_layernorm)"""
         x = h16 if h16 is not None else h
         T, R = ctx.T, ctx.T * self.top
         logits = so.linear(x, self.router, self.router_b, math=so.MATH_F32 if ctx.math == so.MATH_F32 else so.MATH_F32_STREAM)
@@ -444,6 +446,8 @@ class ExpertMlp:
             gu = so.linear_segmented(x, self.w_up, seg, src_row, T, R, math=ctx.math)
             y = so.moe_glu(gu, self.F, self.limit, GLU_SLOPE, ctx_rows(ctx, R, self.F), unit=self.unit)
         d = so.linear_segmented(y, self.w_down, seg, None, T, R, math=ctx.math)
+        if defer and not self.identity and self.shared is None:
+            return d, dst, wts
         add = self.shared(ctx, h, h16) if self.shared is not None else None
         return so.moe_combine(d, dst, wts, T, self.top, ids=ids if self.identity else None, n_real=self.E, own=x, add=add)
 

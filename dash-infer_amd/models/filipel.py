@@ -117,9 +117,13 @@ class Filipel:
         for i, (_, mixer, ff) in enumerate(self.layers):
             h32, h16 = (None, h) if act == torch.bfloat16 else (h, None)
             mo = mixer(ctx, h32, h16)
-            fo = ff(ctx, h32, h16) if ff is not None else None
+            fo = routed = None
+            if isinstance(ff, mixers.ExpertMlp):      # its weighted sum over the experts joins the residual step
+                routed = ff(ctx, h32, h16, defer=True)
+            elif ff is not None:
+                fo = ff(ctx, h32, h16)
             nxt = self.layers[i + 1][0] if i + 1 < len(self.layers) else None
-            h = so.residual_layernorm(x, nxt, a=mo, b=fo, mult=self.mult, eps=self.eps, x_out=x, out_dtype=act)
+            h = so.residual_layernorm(x, nxt, a=mo, b=fo, routed=routed, mult=self.mult, eps=self.eps, x_out=x, out_dtype=act)
             if ctx.taps is not None:
                 ctx.taps[i] = x.clone()
         return x

@@ -85,10 +85,12 @@ class Vabanex:
     def second_rows(self, prev, tokens):
         return None      # one embedding table
 
-    def _residual(self, x, norm, a=None):
-        """x += a; the layer norm of the result for what comes next (None: no norm), one launch"""
+    def _residual(self, x, norm, y=None):
+        """x += y (the rows of a sublayer, or the parts of a routed feed-forward's sum); the layer norm of the result for what comes next
+        (None: no norm), one launch"""
         w, b = norm if norm is not None else (None, None)
-        return so.residual_layernorm(x, w, a=a, eps=self.eps, x_out=x if a is not None else None, bias=b, out_dtype=self.act_dtype)
+        a, routed = (None, y) if isinstance(y, tuple) else (y, None)
+        return so.residual_layernorm(x, w, a=a, routed=routed, eps=self.eps, x_out=x if y is not None else None, bias=b, out_dtype=self.act_dtype)
 
     def forward(self, ctx):
         """-> the residual stream after the last layer, [T, width] f32.  A sublayer's residual step and the next sublayer's input norm
@@ -100,7 +102,8 @@ class Vabanex:
             nxt = self.layers[i + 1][0] if i + 1 < len(self.layers) else None
             mo = mixer(ctx, *split(h))
             if ff is not None:
-                mo = ff(ctx, *split(self._residual(x, norm2, mo)))
+                h = self._residual(x, norm2, mo)
+                mo = ff(ctx, *split(h), **({"defer": True} if isinstance(ff, mixers.ExpertMlp) else {}))
             h = self._residual(x, nxt, mo)
             if ctx.taps is not None:
                 ctx.taps[i] = x.clone()

@@ -53,7 +53,7 @@ _SIGS = {
     "dihip_seq_moe_route": (i32, [vp, vp, lng, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, vp, i32, i32, i32, i32, i32, f32]),
     "dihip_seq_moe_glu": (i32, [vp, vp, i32, lng, vp, lng, i32, i32, f32, f32, i32]),
     "dihip_seq_moe_combine": (i32, [vp, vp, lng, vp, lng, vp, vp, i32, i32, i32, vp, i32, vp, i32, lng, vp, lng]),
-    "dihip_residual_layernorm": (i32, [vp, vp, vp, vp, lng, vp, lng, f32, vp, vp, vp, i32, f32, vp, i32, lng, i32, i32]),
+    "dihip_residual_layernorm": (i32, [vp, vp, vp, vp, lng, vp, lng, vp, lng, vp, vp, i32, f32, vp, vp, vp, i32, f32, vp, i32, lng, i32, i32]),
     "dihip_polynorm": (i32, [vp, vp, i32, lng, vp, lng, vp, i32, f32, i32, i32]),
     "dihip_rmsnorm_pair": (i32, [vp, vp, lng, vp, lng, vp, vp, lng, vp, i32, f32, f32, i32, i32]),
     "dihip_gate_group_rmsnorm": (i32, [vp, vp, i32, lng, vp, lng, vp, lng, vp, vp, lng, vp, i32, f32, i32, i32, i32, i32]),

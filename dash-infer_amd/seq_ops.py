@@ -370,16 +370,21 @@ def moe_combine(rows, dst, wts, T, top, out=None, ids=None, n_real=0, own=None, 
     return o
 
 
-def residual_layernorm(x_in, w=None, a=None, b=None, mult=1.0, eps=1e-5, x_out=None, row_idx=None, bias=None, out_dtype=torch.float32):
+def residual_layernorm(x_in, w=None, a=None, b=None, mult=1.0, eps=1e-5, x_out=None, row_idx=None, bias=None, out_dtype=torch.float32,
+                       routed=None):
     """x_out = x_in + mult * (a + b);  h = layer_norm(x_out) * w (+ bias)  (mean and variance over the row) -> h (None without w).
+    routed: (rows, dst, wts [T, top]) of a routed feed-forward, whose weighted sum per token (moe_combine) joins a + b.
     row_idx: the norm of the chosen rows of x_in alone."""
     K = x_in.shape[1]
     M = x_in.shape[0] if row_idx is None else row_idx.shape[0]
     assert x_in.is_contiguous() and x_in.dtype == torch.float32 and (x_out is None or x_out.is_contiguous())
-    assert a is None or x_out is not None
+    assert (a is None and routed is None) or x_out is not None
+    rows, dst, wts = routed if routed is not None else (None, None, None)
+    assert routed is None or (rows.dtype == wts.dtype == torch.float32 and rows.shape[1] == K and wts.shape[0] == M and wts.is_contiguous())
     h = torch.empty(M, K, dtype=out_dtype, device=x_in.device) if w is not None else None
     check(lib().dihip_residual_layernorm(stream(), ptr(x_out), ptr(x_in), ptr(a), _rows(a) if a is not None else 0, ptr(b),
-                                         _rows(b) if b is not None else 0, float(mult), ptr(row_idx), ptr(w), ptr(bias),
+                                         _rows(b) if b is not None else 0, ptr(rows), _rows(rows) if rows is not None else 0, ptr(dst), ptr(wts),
+                                         wts.shape[1] if wts is not None else 0, float(mult), ptr(row_idx), ptr(w), ptr(bias),
                                          dt(w) if w is not None else F32_CODE, float(eps), ptr(h), dt(h) if h is not None else F32_CODE,
                                          _rows(h) if h is not None else 0, M, K), "dihip_residual_layernorm")
     return h

@@ -175,7 +175,13 @@ def operator_table(size, prompt_len, like=False):
         add(f"experts' {'[gate | up] product + silu unit' if like else 'up product + gelu'} {P} pairs x {F}", units, 2.0 * P * n_up * W, 2.0 * used * n_up * W + 2.0 * P * (W + F))
         add(f"experts' down product {P} pairs", lambda: so.linear_segmented(y, w_dn, seg, None, T, P, out=d, math=so.MATH_BF16), 2.0 * P * F * W,
             2.0 * used * F * W + 2.0 * P * F + 4.0 * P * W)
-        add(f"weighted sum of the experts T={T}", lambda: so.moe_combine(d, dst, wts, T, top), 0, 4.0 * P * W + 4.0 * T * W)
+        if like:
+            add(f"residual of a sublayer + {top} routed rows per token + layer norm T={T}",
+                lambda: so.residual_layernorm(x, nw, a=m1, routed=(d, dst, wts), mult=0.5, eps=1e-6, x_out=x, out_dtype=torch.bfloat16), 0,
+                4.0 * P * W + 14.0 * T * W)
+        else:
+            add(f"residual of {top} routed rows per token + biased layer norm T={T}",
+                lambda: so.residual_layernorm(x, nw, routed=(d, dst, wts), eps=1e-6, x_out=x, bias=nb, out_dtype=torch.bfloat16), 0, 4.0 * P * W + 10.0 * T * W)
         if T == 1:
             head = bf(s["vocab"], W)
             add(f"head {'' if like else '+ cap '}{s['vocab']} x {W}", lambda: so.linear(h16, head, act=None if like else "softcap", act_param=20.0, math=so.MATH_BF16),

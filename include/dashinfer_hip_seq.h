@@ -60,12 +60,13 @@ int dihip_add_dyt(void* stream, float* x_out, const float* x_in, const float* a,
                   int M, int K);
 
 /* Layers that run their sublayers side by side on a layer-normed stream: the residual step and the NEXT input norm in one launch,
- *   x_out[r] = x_in[r] + mult * (a[r] + b[r])   (a NULL: x_in itself; b NULL: a alone),
+ *   x_out[r] = x_in[r] + mult * (a[r] + b[r] + sum_k wts[r, k] * rows[dst[r * top + k]])
+ *              (each part may be absent: a NULL, b NULL (b goes with a), dst NULL; the sum is dihip_seq_moe_combine's; none: x_in itself),
  *   h[i] = (x_out[r] - mean) / sqrt(var + eps) * w (+ bias)   (mean and variance over the row; bias NULL: none; w NULL: no norm)
  * r = row_idx ? row_idx[i] : i (with row_idx x_out must be NULL).  x_in / x_out: contiguous [., K] f32 (may alias); h: rows of
  * stride ldh, f32 or bf16. */
 int dihip_residual_layernorm(void* stream, float* x_out, const float* x_in, const float* a, long lda, const float* b, long ldb,
-                             float mult, const int32_t* row_idx, const void* w, const void* bias, int w_dtype, float eps, void* h,
+                             const float* rows, long ldr, const int32_t* dst, const float* wts, int top, float mult, const int32_t* row_idx, const void* w, const void* bias, int w_dtype, float eps, void* h,
                              int h_dtype, long ldh, int M, int K);
 /* y[t] = c0 z / rms(z) + c1 z^2 / rms(z^2) + c2 z^3 / rms(z^3) + c3,  powers per element, rms(v) = sqrt(mean(v^2) + eps) over the
  * F elements of the row; coef = (c0, c1, c2, c3) of w_dtype */

@@ -58,6 +58,24 @@ def test_biased_layer_norm_fused_with_the_residual_step(so, K):
     assert rel_err(hr.cpu().numpy(), ov.layer_norm(x, w, 0.0 * b, 1e-4)[pick]) > 1e-2      # the bias shows
 
 
+@pytest.mark.parametrize("K", [72, 3000, 17000])
+@pytest.mark.parametrize("top", [1, 3])
+def test_routed_rows_summed_inside_the_residual_step(so, K, top):
+    """the bits of the separate sum, beside another sublayer's rows or alone"""
+    rng = np.random.default_rng(2)
+    T = 9
+    x, a, rows = (rng.normal(0, 1.0, (n, K)).astype(np.float32) for n in (T, T, T * top))
+    wts, dst = rng.uniform(0, 2, (T, top)).astype(np.float32), rng.permutation(T * top)
+    w, b = dev(bf(1.0 + 0.3 * rng.normal(size=K))), dev(bf(rng.normal(size=K)))
+    y = so.moe_combine(dev(rows), i32(dst), dev(wts), T, top)
+    assert rel_err(y.cpu().numpy(), (wts[:, :, None] * rows[dst].reshape(T, top, K).astype(np.float64)).sum(1)) < 1e-6
+    for other in (None, dev(a)):
+        x1, x2 = dev(x), dev(x)
+        h1 = so.residual_layernorm(x1, w, a=other if other is not None else y, b=y if other is not None else None, mult=0.5, eps=1e-5, x_out=x1, bias=b)
+        h2 = so.residual_layernorm(x2, w, a=other, routed=(dev(rows), i32(dst), dev(wts)), mult=0.5, eps=1e-5, x_out=x2, bias=b)
+        assert torch.equal(x1, x2) and torch.equal(h1, h2)
+
+
 def test_scaled_embedding_rows(so):
     rng = np.random.default_rng(1)
     table = bf(rng.normal(size=(37, 50)))

@@ -311,6 +311,27 @@ def test_latent_attention_whose_value_is_a_part_of_the_row(so, R, RV, H, window,
         assert rel_err(row.cpu().numpy(), want) < 2e-5, (start, count)
 
 
+@pytest.mark.parametrize("R,RV", [(64, 64), (576, 512)])
+def test_latent_attention_over_more_pages_than_are_staged(so, R, RV):
+    """walks over more span pointers than a workgroup keeps in LDS: one key that stands out behind them, at the start, and near the end"""
+    rng = np.random.default_rng(R)
+    n, H = 9000, 2
+    rows = torch.from_numpy(rng.normal(0, 0.3, (n, R)).astype(np.float32)).to(torch.bfloat16).float().numpy()
+    q = rng.normal(0, 1, R).astype(np.float32)
+    i32 = lambda a: torch.tensor(a, dtype=torch.int32).cuda()
+    for at in (3, 8300, 8990):
+        r = rows.copy()
+        r[at] = torch.from_numpy(4.0 * q / np.linalg.norm(q) * 3.0).to(torch.bfloat16).float().numpy()
+        st, tab, slot = filled_cache(r, torch.bfloat16)
+        pos = [n - 3, n - 2, n - 1]
+        qr = torch.from_numpy(np.tile(q, (3, H))).to(torch.bfloat16).float().numpy()
+        want = attn_ref(qr, r, pos, H, 0, 0.3, None).reshape(3, H, R)[:, :, :RV].reshape(3, H * RV)
+        assert rel_err(want[0, :RV], r[at, :RV]) < 0.2
+        for nsplit in (1, 2):
+            got = so.latent_window_attn_mc(dev(qr), tab, None, i32(pos), i32([slot.index]), i32([0]), i32([3]), 3, n - 1, H, 0, 0.3, nsplit=nsplit, value=RV)
+            assert rel_err(got.cpu().numpy(), want) < 8e-3, (at, nsplit)
+
+
 def test_gated_recurrence_in_chunks_side_by_side(so):
     """long portions cut into chunks that run in parallel: two portions of unequal length (one shorter than a chunk) that start
     from states an earlier step left"""

@@ -212,20 +212,32 @@ __global__ __launch_bounds__(256) void gla_carry_kernel(GlaArgs a) {
   }
 }
 
+// y = x * div[t, h] / rms(x * div[t, h]) * gamma * mul * out_scale per head; gamma [DV] shared by the heads (gamma_stride 0), [H * DV]
+// (gamma_stride DV) or absent; div absent: 1
+struct HeadNormArgs {
+  void* y; int ydt; long ldy;
+  const float* x; long ldx;
+  const void* gamma; int gamma_stride; float eps;
+  const float* div; const float* mul; long ldm;
+  float out_scale; int H, DV;
+};
 template <int WT>
-__global__ __launch_bounds__(256) void head_rmsnorm_mul_kernel(void* __restrict__ y, int ydt, long ldy, const float* __restrict__ x, long ldx,
-                                                               const void* __restrict__ gamma, float eps, const float* __restrict__ mul,
-                                                               long ldm, int H, int DV) {
-  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  for (int h = blockIdx.y * 4 + wave; h < H; h += 4 * gridDim.y) {
-    const float* xr = x + (size_t)t * ldx + (size_t)h * DV;
+__global__ __launch_bounds__(256) void head_rmsnorm_mul_kernel(HeadNormArgs a) {
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, DV = a.DV;
+  for (int h = blockIdx.y * 4 + wave; h < a.H; h += 4 * gridDim.y) {
+    const float* xr = a.x + (size_t)t * a.ldx + (size_t)h * DV;
+    const float f = a.div ? a.div[(size_t)t * a.H + h] : 1.f;
     float ss = 0.f;
-    for (int d = lane; d < DV; d += 64) ss = __builtin_fmaf(xr[d], xr[d], ss);
-    const float inv = 1.f / sqrtf(wave_sum(ss) / (float)DV + eps);
     for (int d = lane; d < DV; d += 64) {
-      float v = xr[d] * inv * load_ft<WT>(gamma, d);
-      if (mul) v *= mul[(size_t)t * ldm + (size_t)h * DV + d];
-      st_any(y, (size_t)t * ldy + (size_t)h * DV + d, ydt, v);
+      const float v = xr[d] * f;
+      ss = __builtin_fmaf(v, v, ss);
+    }
+    const float inv = 1.f / sqrtf(wave_sum(ss) / (float)DV + a.eps);
+    for (int d = lane; d < DV; d += 64) {
+      float v = xr[d] * f * inv;
+      if (a.gamma) v *= load_ft<WT>(a.gamma, (size_t)h * a.gamma_stride + d);
+      if (a.mul) v *= a.mul[(size_t)t * a.ldm + (size_t)h * DV + d];
+      st_any(a.y, (size_t)t * a.ldy + (size_t)h * DV + d, a.ydt, v * a.out_scale);
     }
   }
 }
@@ -321,15 +333,16 @@ int dihip_ssd(void* stream, float* out, long ldo, const float* x, long ldx, cons
   return launch_status();
 }
 
-int dihip_head_rmsnorm_mul(void* stream, void* y, int y_dtype, long ldy, const float* x, long ldx, const void* gamma, int w_dtype,
-                           float eps, const float* mul, long ldm, int T, int H, int DV) {
-  DIHIP_REQUIRE(T >= 0 && H > 0 && DV > 0 && y && x && gamma && ldy >= (long)H * DV && ldx >= (long)H * DV && (!mul || ldm >= (long)H * DV) &&
+int dihip_head_rmsnorm_mul(void* stream, void* y, int y_dtype, long ldy, const float* x, long ldx, const void* gamma, int gamma_per_head, int w_dtype,
+                           float eps, const float* div, const float* mul, long ldm, float out_scale, int T, int H, int DV) {
+  DIHIP_REQUIRE(T >= 0 && H > 0 && DV > 0 && y && x && ldy >= (long)H * DV && ldx >= (long)H * DV && (!mul || ldm >= (long)H * DV) &&
                     seq_dtype_ok(y_dtype) && seq_dtype_ok(w_dtype), DIHIP_PARAM_ERROR, "head_rmsnorm_mul: bad argument");
   if (T == 0) return DIHIP_SUCCESS;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   const dim3 grid(T, T >= 256 ? 1 : (H + 3) / 4);   // few rows (decoding): a wave per head; many rows: a workgroup per row
-  if (w_dtype == DIHIP_F32) hipLaunchKernelGGL(head_rmsnorm_mul_kernel<DIHIP_F32>, grid, dim3(256), 0, s, y, y_dtype, ldy, x, ldx, gamma, eps, mul, ldm, H, DV);
-  else hipLaunchKernelGGL(head_rmsnorm_mul_kernel<DIHIP_BF16>, grid, dim3(256), 0, s, y, y_dtype, ldy, x, ldx, gamma, eps, mul, ldm, H, DV);
+  const HeadNormArgs a{y, y_dtype, ldy, x, ldx, gamma, gamma_per_head ? DV : 0, eps, div, mul, ldm, out_scale, H, DV};
+  if (w_dtype == DIHIP_F32) hipLaunchKernelGGL(head_rmsnorm_mul_kernel<DIHIP_F32>, grid, dim3(256), 0, s, a);
+  else hipLaunchKernelGGL(head_rmsnorm_mul_kernel<DIHIP_BF16>, grid, dim3(256), 0, s, a);
   return launch_status();
 }
 

@@ -2,6 +2,8 @@
 //   qkv_prep_append   per token: unit-RMS norm of every query / key head (optional), rotary positions (paired or half-split
 //                     layout, a frequency table and a magnitude from the host), mixing of the values with another layer's,
 //                     queries written back in place, keys and values appended to their pages
+//   qkv_conv_prep_append   the same for a layer with a short causal convolution on every channel of q, k and v and norms over the
+//                     whole query / key row
 //   gqa_attn_kernel   one workgroup per row, every product and sum in f32 (any cache type)
 //   gqa_attn_mc_kernel + merge   bf16 caches on the matrix cores, the key walk split for few rows (decoding)
 // Options of the softmax: a sink logit per head or the constant 0 (one more term in the denominator, no value), a tanh cap on
@@ -98,6 +100,76 @@ __global__ __launch_bounds__(256) void qkv_prep_append_kernel(PrepArgs a) {
   }
 }
 
+// ------------------------------------------------------------------------------------------------ convolution + prep + append
+// u[c] = sum_j w[c, j] x[t - (taps - 1) + j, c] for the channels [q | k | v] of the rows x (inputs of earlier steps: the slot's tail), then
+// the query row and the key row as a whole are divided by their root mean square and weighted, their heads rotated; queries go to q_out,
+// keys and values to their pages.  A workgroup per (row, q / k / v); the convolved row is kept in LDS.
+struct ConvPrepArgs {
+  const float* x; long ld;                     // [T][HD + GD + GV]
+  const void* w; const void* qnorm; const void* knorm; int wdt; int taps;
+  float* tail; int write_tail;                 // [slots][taps - 1][C]; write_tail: every portion has ONE row, which also moves its tail on
+  float eps; const float* freq; int rot_dims, pairs; float mag;
+  float* q_out; long ldq;
+  void* const* kspans; void* const* vspans; int span_stride, span_len, cdt;
+  const int32_t* tok_slot; const int32_t* tok_pos; const int32_t* tok_off;
+  int HD, GD, GV, D;
+};
+
+template <int NT>
+__global__ __launch_bounds__(NT) void qkv_conv_prep_append_kernel(ConvPrepArgs a) {
+  extern __shared__ float us[];
+  __shared__ float cs[128], sn[128], red[NT / 64];
+  const int t = blockIdx.x, part = blockIdx.y, tid = threadIdx.x;      // part 0: q, 1: k, 2: v
+  const int pos = a.tok_pos[t], off = a.tok_off[t], nt = a.taps - 1, C = a.HD + a.GD + a.GV, half = a.rot_dims >> 1;
+  const int c0 = part == 0 ? 0 : (part == 1 ? a.HD : a.HD + a.GD), n = part == 0 ? a.HD : (part == 1 ? a.GD : a.GV);
+  const size_t sp = (size_t)a.tok_slot[t] * a.span_stride + pos / a.span_len, in_span = (size_t)(pos % a.span_len);
+  float* tl = a.tail ? a.tail + (size_t)a.tok_slot[t] * nt * C : nullptr;
+  if (part < 2)
+    for (int i = tid; i < half; i += NT) {
+      float s, c;
+      rope_sincos((uint32_t)pos, a.freq[i], &s, &c);
+      sn[i] = s * a.mag;
+      cs[i] = c * a.mag;
+    }
+  float ss = 0.f;
+  for (int i = tid; i < n; i += NT) {
+    const int c = c0 + i;
+    float acc = 0.f;
+    for (int k = 0; k < a.taps; ++k) {
+      const int d = nt - k, o = off - d;
+      const float v = o >= 0 ? a.x[(size_t)(t - d) * a.ld + c] : tl[(size_t)(nt + o) * C + c];
+      acc = __builtin_fmaf(ld_any(a.w, (size_t)c * a.taps + k, a.wdt), v, acc);
+      if (a.write_tail && k > 0) tl[(size_t)(k - 1) * C + c] = v;      // (off == 0: row k - 1 was read in the turn before)
+    }
+    ss = __builtin_fmaf(acc, acc, ss);
+    if (part < 2) us[i] = acc;
+    else st_any(a.vspans[sp], in_span * n + i, a.cdt, acc);
+  }
+  if (part == 2) return;
+  ss = wave_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  ss = 0.f;
+#pragma unroll
+  for (int w = 0; w < NT / 64; ++w) ss += red[w];
+  const float inv = 1.f / sqrtf(ss / (float)n + a.eps);
+  const void* gamma = part == 0 ? a.qnorm : a.knorm;
+  void* kdst = part == 1 ? a.kspans[sp] : nullptr;
+  auto normed = [&](int i) { return gamma ? us[i] * inv * ld_any(gamma, i, a.wdt) : us[i]; };
+  for (int i = tid; i < n; i += NT) {
+    const int d = i % a.D;
+    float y = normed(i);
+    if (d < a.rot_dims) {
+      const int p = a.pairs ? d >> 1 : (d < half ? d : d - half);
+      const bool first = a.pairs ? (d & 1) == 0 : d < half;
+      const float o = normed(a.pairs ? (first ? i + 1 : i - 1) : (first ? i + half : i - half));
+      y = first ? y * cs[p] - o * sn[p] : y * cs[p] + o * sn[p];
+    }
+    if (part == 0) a.q_out[(size_t)t * a.ldq + i] = y;
+    else st_any(kdst, in_span * n + i, a.cdt, y);
+  }
+}
+
 // ------------------------------------------------------------------------------------------------ f32 row kernel
 struct GqaArgs {
   float* out; long ldo;
@@ -105,7 +177,7 @@ struct GqaArgs {
   void* const* kspans; void* const* vspans; int span_stride, span_len;
   const void* sink; int wdt, sink_mode;   // 0: none, 1: sink[h], 2: the constant 0
   float softcap;                          // <= 0: none
-  const float* gate; long ldg;            // [T, H] multiplier (NULL: none)
+  const float* gate; long ldg;            // [T, H] multiplier (NULL: none; ldg 0: one row for all)
   const int32_t* tok_slot; const int32_t* tok_pos; const int32_t* ent_slot; const int32_t* ent_row0; const int32_t* ent_count;
   int H, G, D, DV; float scale;
   float* ws; int rows_total;
@@ -507,13 +579,35 @@ int dihip_qkv_prep_append(void* stream, float* qkv, long ld, int q_off, int k_of
   return launch_status();
 }
 
+int dihip_qkv_conv_prep_append(void* stream, const float* x, long ld, const void* conv, int taps, float* tail, int write_tail, int H, int G, int D,
+                               int DV, const void* qnorm, const void* knorm, int w_dtype, float eps, const float* freq, int rot_dims, int layout,
+                               float mag, float* q_out, long ldq, void* const* kspans, void* const* vspans, int span_stride, int span_len,
+                               int cache_dtype, const int32_t* tok_slot, const int32_t* tok_pos, const int32_t* tok_off, int T) {
+  DIHIP_REQUIRE(T >= 0 && x && conv && H > 0 && G > 0 && H % G == 0 && D > 0 && DV > 0 && q_out && kspans && vspans && tok_slot && tok_pos && tok_off &&
+                    span_stride > 0 && span_len > 0 && seq_dtype_ok(cache_dtype) && seq_dtype_ok(w_dtype), DIHIP_PARAM_ERROR,
+                "qkv_conv_prep_append: bad argument");
+  DIHIP_REQUIRE(taps >= 1 && taps <= 16 && (tail || taps == 1), DIHIP_PARAM_ERROR, "qkv_conv_prep_append: 1 to 16 taps, with their state");
+  DIHIP_REQUIRE(ld >= (long)(H + G) * D + (long)G * DV && ldq >= (long)H * D, DIHIP_PARAM_ERROR, "qkv_conv_prep_append: columns outside the rows");
+  DIHIP_REQUIRE(rot_dims >= 0 && rot_dims <= D && rot_dims <= 256 && rot_dims % 2 == 0 && (rot_dims == 0 || freq) && (layout == 0 || layout == 1),
+                DIHIP_PARAM_ERROR, "qkv_conv_prep_append: bad rotation (an even number of at most 256 dimensions up to the head size, layout 0 / 1)");
+  DIHIP_REQUIRE((long)H * D <= 15360, DIHIP_EXCEED_LIMIT_ERROR, "qkv_conv_prep_append: query rows of more than 15360 elements");
+  if (T == 0) return DIHIP_SUCCESS;
+  ConvPrepArgs a{x, ld, conv, qnorm, knorm, w_dtype, taps, taps > 1 ? tail : nullptr, write_tail && taps > 1, eps, freq, rot_dims, layout == 0, mag, q_out, ldq,
+                 kspans, vspans, span_stride, span_len, cache_dtype, tok_slot, tok_pos, tok_off, H * D, G * D, G * DV, D};
+  const size_t lds = (size_t)H * D * sizeof(float);      // (G <= H: the key row fits too)
+  hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+  if (H * D <= 1024) hipLaunchKernelGGL(qkv_conv_prep_append_kernel<256>, dim3(T, 3), dim3(256), lds, s, a);
+  else hipLaunchKernelGGL(qkv_conv_prep_append_kernel<1024>, dim3(T, 3), dim3(1024), lds, s, a);
+  return launch_status();
+}
+
 static int gqa_check(const char* what, const float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
                      int span_stride, int span_len, const void* sink, int w_dtype, int sink_mode, const float* gate, long ldg, int H, int G,
                      int D, int DV, int maps, int keep_first) {
   DIHIP_REQUIRE(maps >= 1 && maps <= 8 && keep_first >= 0, DIHIP_PARAM_ERROR, "%s: 1 to 8 maps per head, no negative count of kept keys", what);
   DIHIP_REQUIRE(out && q && kspans && vspans && span_stride > 0 && span_len > 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && DV > 0 &&
                     ldo >= (long)H * maps * DV && ldq >= (long)H * maps * D && seq_dtype_ok(w_dtype), DIHIP_PARAM_ERROR, "%s: bad argument", what);
-  DIHIP_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 1 || sink) && (!gate || ldg >= H), DIHIP_PARAM_ERROR,
+  DIHIP_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 1 || sink) && (!gate || ldg >= H || ldg == 0), DIHIP_PARAM_ERROR,
                 "%s: bad sink mode or gate", what);
   return DIHIP_SUCCESS;
 }

@@ -1,6 +1,8 @@
 // seq_norms.hip -- row operators of layers that run their sublayers side by side on a layer-normed stream (everything in f32):
 //   residual_layernorm   x_out = x_in + mult * (a + b + routed experts' weighted rows);  h = (x_out - mean) / sqrt(var + eps) * w (+ bias)  -- the residual step of
 //                        two sublayers and the NEXT layer's input norm in one launch; with row_idx: the norm of chosen rows alone
+//   residual_rmsnorm     x_out = x_in + (a + b + bias + routed experts' weighted rows) + again;  h1, h2 = x_out / rms(x_out) * (add + w1 / w2)
+//                        * scale -- the same step for RMS norms, one statistic for the two input norms of the next layer's sublayers
 //   polynorm             y = c0 z / rms(z) + c1 z^2 / rms(z^2) + c2 z^3 / rms(z^3) + c3   (powers per element, rms over the row)
 //   rmsnorm_pair         y = coef * (xa / rms(xa) * wa + xb / rms(xb) * wb)   -- two branches joined on equal footing
 //   gate_group_rmsnorm   v = (o + skip[head] * x) * silu(z);  y = v / rms_group(v) * w   -- the gate comes before the norm, the norm
@@ -63,6 +65,44 @@ __global__ __launch_bounds__(256) void residual_layernorm_kernel(float* x_out, c
     float y = (src[k] - mean) * inv * load_ft<WT>(w, k);
     if (bias) y += load_ft<WT>(bias, k);
     st_any(h, (size_t)i * ldh + k, hdt, y);
+  }
+}
+
+// The residual step of two sublayers that run side by side with an input norm EACH: both norms divide by the same root mean square.
+struct ResidualRms {
+  float* x_out; const float* x_in;
+  const float* a; long lda; const float* b; long ldb; const float* bias; const float* again; long ldagain;
+  RoutedRows q;
+  const int32_t* row_idx;
+  const void* w1; const void* w2; float add, scale, eps;
+  void* h1; void* h2; int hdt; long ldh;
+  int K;
+};
+template <int WT>
+__global__ __launch_bounds__(256) void residual_rmsnorm_kernel(ResidualRms p) {
+  __shared__ float red[4];
+  const int i = blockIdx.x, K = p.K;
+  const size_t r = p.row_idx ? (size_t)p.row_idx[i] : (size_t)i;
+  float ss = 0.f;
+#pragma unroll 4
+  for (int k = threadIdx.x; k < K; k += 256) {
+    float s = p.a ? p.a[r * p.lda + k] : 0.f;
+    if (p.b) s += p.b[r * p.ldb + k];
+    if (p.bias) s += p.bias[k];
+    if (p.q.dst) s += routed_sum(p.q, r, k);
+    float v = p.x_in[r * K + k] + s;
+    if (p.again) v += p.again[r * p.ldagain + k];
+    if (p.x_out) p.x_out[r * K + k] = v;     // (re-read below by the thread that wrote it)
+    ss = __builtin_fmaf(v, v, ss);
+  }
+  if (!p.w1 && !p.w2) return;
+  const float* src = p.x_out ? p.x_out + r * K : p.x_in + r * K;
+  const float inv = 1.f / sqrtf(block256_sum(ss, red) / (float)K + p.eps);
+#pragma unroll 4
+  for (int k = threadIdx.x; k < K; k += 256) {
+    const float v = src[k] * inv;
+    if (p.w1) st_any(p.h1, (size_t)i * p.ldh + k, p.hdt, v * (p.add + load_ft<WT>(p.w1, k)) * p.scale);
+    if (p.w2) st_any(p.h2, (size_t)i * p.ldh + k, p.hdt, v * (p.add + load_ft<WT>(p.w2, k)) * p.scale);
   }
 }
 
@@ -227,6 +267,68 @@ __global__ __launch_bounds__(NT) void residual_layernorm_reg_kernel(float* x_out
       float y = (v[e] - mean) * inv * g[e];
       if (bias) y += load_ft<WT>(bias, k);
       st_any(h, (size_t)i * ldh + k, hdt, y);
+    }
+  }
+}
+
+template <int WT, int NT, int EPT>
+__global__ __launch_bounds__(NT) void residual_rmsnorm_reg_kernel(ResidualRms p) {
+  __shared__ float red[NT / 64];
+  const int i = blockIdx.x, tid = threadIdx.x, K = p.K;
+  const size_t r = p.row_idx ? (size_t)p.row_idx[i] : (size_t)i;
+  float v[EPT], s[EPT], g1[EPT], g2[EPT];
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) {
+    const int k = min(tid + e * NT, K - 1);
+    v[e] = p.x_in[r * K + k];
+    s[e] = p.a ? p.a[r * p.lda + k] : 0.f;
+    g1[e] = p.w1 ? load_ft<WT>(p.w1, k) : 0.f;
+    g2[e] = p.w2 ? load_ft<WT>(p.w2, k) : 0.f;
+  }
+  if (p.b) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) s[e] += p.b[r * p.ldb + min(tid + e * NT, K - 1)];
+  }
+  if (p.bias) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) s[e] += p.bias[min(tid + e * NT, K - 1)];
+  }
+  if (p.q.dst) {
+    float acc[EPT];
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) acc[e] = 0.f;
+    for (int j = 0; j < p.q.top; ++j) {
+      const float wt = p.q.wts[r * p.q.top + j];
+      const float* row = p.q.rows + (size_t)p.q.dst[r * p.q.top + j] * p.q.ld;
+#pragma unroll
+      for (int e = 0; e < EPT; ++e) acc[e] = __builtin_fmaf(wt, row[min(tid + e * NT, K - 1)], acc[e]);
+    }
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) s[e] += acc[e];
+  }
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) v[e] += s[e];
+  if (p.again) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) v[e] += p.again[r * p.ldagain + min(tid + e * NT, K - 1)];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) {
+    const int k = tid + e * NT;
+    if (k < K) {
+      if (p.x_out) p.x_out[r * K + k] = v[e];
+      ss = __builtin_fmaf(v[e], v[e], ss);
+    }
+  }
+  if (!p.w1 && !p.w2) return;
+  const float inv = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)K + p.eps);
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) {
+    const int k = tid + e * NT;
+    if (k < K) {
+      if (p.w1) st_any(p.h1, (size_t)i * p.ldh + k, p.hdt, v[e] * inv * (p.add + g1[e]) * p.scale);
+      if (p.w2) st_any(p.h2, (size_t)i * p.ldh + k, p.hdt, v[e] * inv * (p.add + g2[e]) * p.scale);
     }
   }
 }
@@ -421,6 +523,21 @@ int dihip_residual_layernorm(void* stream, float* x_out, const float* x_in, cons
   if (M == 0) return DIHIP_SUCCESS;
   BY_WT_ROW(residual_layernorm, K, w_dtype, dim3(M), reinterpret_cast<hipStream_t>(stream), x_out, x_in, a, lda, b, ldb,
             (RoutedRows{rows, ldr, dst, wts, top}), mult, row_idx, w, bias, eps, h, h_dtype, ldh, K);
+  return launch_status();
+}
+
+int dihip_residual_rmsnorm(void* stream, float* x_out, const float* x_in, const float* a, long lda, const float* b, long ldb, const float* bias,
+                           const float* again, long ldagain, const float* rows, long ldr, const int32_t* dst, const float* wts, int top,
+                           const int32_t* row_idx, const void* w1, const void* w2, int w_dtype, float add, float scale, float eps, void* h1, void* h2,
+                           int h_dtype, long ldh, int M, int K) {
+  DIHIP_REQUIRE(M >= 0 && K > 0 && x_in && (!a || lda >= K) && (!b || ldb >= K) && (!again || ldagain >= K) && (!w1 || (h1 && ldh >= K)) &&
+                    (!w2 || (h2 && ldh >= K)) && (!row_idx || !x_out) && (x_out || (!a && !b && !bias && !again && !dst)) && seq_dtype_ok(w_dtype) &&
+                    seq_dtype_ok(h_dtype), DIHIP_PARAM_ERROR, "residual_rmsnorm: bad argument");
+  DIHIP_REQUIRE(!dst || (rows && wts && top > 0 && ldr >= K), DIHIP_PARAM_ERROR, "residual_rmsnorm: routed rows need their weights and places");
+  if (M == 0) return DIHIP_SUCCESS;
+  const ResidualRms p{x_out, x_in, a, lda, b, ldb, bias, again, ldagain, RoutedRows{rows, ldr, dst, wts, top}, row_idx, w1, w2, add, scale, eps, h1, h2,
+                      h_dtype, ldh, K};
+  BY_WT_ROW(residual_rmsnorm, K, w_dtype, dim3(M), reinterpret_cast<hipStream_t>(stream), p);
   return launch_status();
 }
 

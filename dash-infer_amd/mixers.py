@@ -16,17 +16,24 @@ to rows of the same shape, reading and updating what its sequences left in the s
                          a sliding window that keeps the first keys of the sequence, two softmax maps per head whose difference
                          is normed per head (differential attention), several runs per step with a cache each (looped layers),
                          a multiplier per head on the scores, softmax maps mixed between the heads after the softmax (talking
-                         heads), a sigmoid gate per output element
+                         heads), a sigmoid gate per output element, a short causal convolution on every channel of queries, keys and
+                         values, a norm over the whole query / key row in place of the heads' own
   GatedLinearAttention   linear attention with a decay per key channel and a matrix state per head (f32, per slot), unit-RMS
                          norm per head, silu output gate
   StateSpaceMixer        state-space duality form: short causal convolution + silu on [x | B | C], a scalar decay per head from a
                          softplus step size, a matrix state per head (f32, per slot), skip term, silu gate BEFORE a grouped RMS norm
+  Retention              linear attention with a constant decay per head and a matrix state (f32, per slot), rotary positions, unit-RMS norm
+                         per head, silu output gate
+  MatrixMemory           mLSTM: a matrix state and a key sum per head (f32, per slot) under exponential input and forget gates held in range
+                         by a running maximum, unit-RMS norm per head, sigmoid output gate
+  WeightedPair           two mixers on the same input, their results added with a constant weight each: one input and one output product
   SideBySide             two mixers on the same input, their results RMS-normed over the width, weighted and averaged
   GatedMlp               down(act(gate(h)) * up(h)); or the clamped sigmoid-gated unit
   ExpertMlp              top-k routed experts; units: clamped sigmoid-gated, silu-gated, or an elementwise activation without a gate;
                          routing: softmax over the chosen logits, or softmax / sigmoid scores with a correction added for the choice
                          alone (weights over their sum or as they are, times a factor), the choice limited to the best groups of
-                         experts; router outputs past the real experts stand for identity experts; an always-on shared expert
+                         experts; router outputs past the real experts stand for identity experts; an always-on shared expert, optionally
+                         with a sigmoid gate per token
 Matrix products run in ctx.math (seq_ops.MATH_F32 / MATH_BF16); norms, scores, gates of the recurrence, decays and
 state are f32 in both.
 """
@@ -182,29 +189,57 @@ class DenseMlp:
 
 
 def rotary_frequencies(dims, base, scaling=None):
-    """frequency per rotated pair (f32 tensor [dims / 2], computed in f64) and the magnitude of cos and sin.  scaling: None or
-    {factor, original, fast, slow}: pairs that turn fewer than `slow` times over `original` positions are slowed down by
-    `factor`, pairs that turn more than `fast` times are kept, a linear ramp over the pair index between; the magnitude grows
-    with 0.1 ln(factor) + 1."""
+    """frequency per rotated pair (f32 tensor [dims / 2], computed in f64) and the magnitude of cos and sin.  scaling: None, or
+      {factor, original, fast, slow}: pairs that turn fewer than `slow` times over `original` positions are slowed down by
+        `factor`, pairs that turn more than `fast` times are kept, a linear ramp over the pair index between; the magnitude grows
+        with 0.1 ln(factor) + 1;
+      {factor, original, low, high}: the same with `low` / `high` turns, the blend between by the number of turns, no magnitude."""
     import math
     f = [float(base) ** (-2.0 * i / dims) for i in range(dims // 2)]
     mag = 1.0
     if scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
-        where = lambda turns: dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(float(base)))
-        lo = max(math.floor(where(float(scaling["fast"]))), 0)
-        hi = min(math.ceil(where(float(scaling["slow"]))), dims - 1)
-        for i in range(dims // 2):
-            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
-            f[i] = f[i] / factor * ramp + f[i] * (1.0 - ramp)
-        mag = 0.1 * math.log(factor) + 1.0
+        if "high" in scaling:
+            low, high = float(scaling["low"]), float(scaling["high"])
+            for i, fi in enumerate(f):
+                turns = orig * fi / (2.0 * math.pi)
+                if turns < low:
+                    f[i] = fi / factor
+                elif turns <= high:
+                    keep = (turns - low) / (high - low) if high > low else 1.0
+                    f[i] = (1.0 - keep) * fi / factor + keep * fi
+        else:
+            where = lambda turns: dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(float(base)))
+            lo = max(math.floor(where(float(scaling["fast"]))), 0)
+            hi = min(math.ceil(where(float(scaling["slow"]))), dims - 1)
+            for i in range(dims // 2):
+                ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+                f[i] = f[i] / factor * ramp + f[i] * (1.0 - ramp)
+            mag = 0.1 * math.log(factor) + 1.0
     return torch.tensor(f, dtype=torch.float64).to(torch.float32), mag
+
+
+def run_names(key, runs):
+    """the cache / state names of a layer that runs `runs` times in a step (a looped layer): one set per run"""
+    return [key] if runs == 1 else [f"{key}.run{r}" for r in range(runs)]
+
+
+def padded_rows(parts):
+    """weight matrices of one input product, each padded with zero rows to a multiple of 4 (its output columns start 16-byte aligned)
+    -> (the rows, the column every part starts at)"""
+    out, lo, at = [], [], 0
+    for p in parts:
+        lo.append(at)
+        pad = -p.shape[0] % 4
+        out += [p] + ([torch.zeros(pad, *p.shape[1:], dtype=p.dtype, device=p.device)] if pad else [])
+        at += p.shape[0] + pad
+    return torch.cat(out, 0).contiguous(), lo
 
 
 class GroupedQueryAttention:
     def __init__(self, key, heads, kv_heads, dim, vdim, scale, w, state, cache_dtype, rot_dims=0, rot_base=10000.0, rot_layout="pairs",
                  rot_scaling=None, qk_norm=False, sink=None, softcap=None, head_gate=False, value_mix=None, window=0, keep_first=0,
-                 differential=None, runs=1, head_temp=None, talk=None, elem_gate=False):
+                 differential=None, runs=1, head_temp=None, talk=None, elem_gate=False, conv=0, out_scale=1.0):
         """w: q [heads*maps*dim, width], k [kv_heads*maps*dim, width], v [kv_heads*vdim, width] (+ q.b / k.b / v.b / o.b where
         present), q.norm / k.norm [dim] (qk_norm), g [heads, width] (head_gate), o [width, heads*vdim].  sink: None, "zero" or a
         tensor [heads].  value_mix: None, ("source", name): this layer's values are kept under `name` for the step, or
@@ -215,8 +250,15 @@ class GroupedQueryAttention:
         runs: how often the layer runs in a step (a looped layer); every run has key and value caches of its own.
         talk [heads, heads]: the heads' softmax maps are mixed after the softmax, w_h <- sum_g talk[h, g] w_g, and head h applies its
         mixed map to the values of its own key/value head; head_temp [heads]: a multiplier per head on the scaled scores;
-        elem_gate: g [heads*vdim, width], the concatenated heads are multiplied by sigmoid(g h) element by element."""
+        elem_gate: g [heads*vdim, width], the concatenated heads are multiplied by sigmoid(g h) element by element.
+        conv > 0: a causal convolution of that many taps on every channel of q, k and v after the projection (w: q.conv / k.conv / v.conv
+        [rows, conv]); qk_norm "row" (with conv): q.norm [heads*dim], k.norm [kv_heads*dim], the norm runs over the whole row.
+        out_scale: a constant on the concatenated heads."""
         assert heads % kv_heads == 0
+        self.taps = int(conv or 0)
+        assert self.taps or qk_norm in (True, False), "a norm over the whole row goes with the convolution"
+        if self.taps:
+            assert qk_norm in ("row", False) and differential is None and value_mix is None and not head_gate and not elem_gate and talk is None
         self.talk = talk.contiguous() if talk is not None else None
         self.head_temp = head_temp.contiguous() if head_temp is not None else None
         self.elem_gate = bool(elem_gate)
@@ -263,7 +305,15 @@ class GroupedQueryAttention:
         self.o, self.o_b = w["o"].contiguous(), w.get("o.b")
         assert self.o.shape[1] == self.H * vdim and w["q"].shape[0] == heads * dim and w["k"].shape[0] == kv_heads * dim
         assert w["v"].shape[0] == self.G * vdim
-        names = [key] if runs == 1 else [f"{key}.run{r}" for r in range(runs)]
+        names = run_names(key, runs)
+        if self.taps:
+            self.conv = torch.cat([w["q.conv"], w["k.conv"], w["v.conv"]], 0).contiguous()
+            assert self.conv.shape == (self.g_lo, self.taps)
+            self.tails = [state.add_state(n + ".tail", (self.taps - 1, self.g_lo)) if self.taps > 1 else None for n in names]
+        self.out_gain, self.out_scale = None, float(out_scale)
+        if float(out_scale) != 1.0:      # a constant output gate: one row for all tokens
+            assert not head_gate and talk is None and differential is None
+            self.out_gain = torch.full((1, self.H), float(out_scale), dtype=torch.float32, device=dev)
         self.ktables = [state.add_span_cache(n + ".k", kv_heads * dim, cache_dtype) for n in names]
         self.vtables = [state.add_span_cache(n + ".v", self.G * vdim, cache_dtype) for n in names]
         self.ktable, self.vtable = self.ktables[0], self.vtables[0]
@@ -273,42 +323,64 @@ class GroupedQueryAttention:
             self.talk32 = self.talk.float().contiguous()
             self.talk_mc = so.talk_attn_mc_supported(self.H, self.G, dim, vdim, self.ktable) and self.n_in % 4 == 0
 
+    @property
+    def act_cols(self):
+        return (self.g_lo, self.n_in) if self.head_gate or self.elem_gate else None
+
     def __call__(self, ctx, h, h16=None, run=0):
+        a = so.linear(h16 if h16 is not None else h, self.w_in, self.b_in, act="sigmoid" if self.act_cols else None, act_cols=self.act_cols,
+                      math=ctx.math)                                        # [q | k | v | gate]
+        return so.linear(self.mix(ctx, a, run), self.o, self.o_b, math=ctx.math)
+
+    def mix(self, ctx, a, run=0, out=None):
+        """a: the input product's rows -> what the output product reads.  out: rows of a wider f32 buffer (or None)"""
         H, G, D, V = self.H, self.G, self.D, self.V
         ktable, vtable = self.ktables[run], self.vtables[run]
-        a = so.linear(h16 if h16 is not None else h, self.w_in, self.b_in, act="sigmoid" if self.head_gate or self.elem_gate else None,
-                      act_cols=(self.g_lo, self.n_in), math=ctx.math)                                        # [q | k | v | gate]
-        vin = vout = None
-        lam = 0.0
-        if self.value_mix is not None:
-            if self.value_mix[0] == "source":
-                vout = ctx.shared[self.value_mix[1]] = torch.empty(ctx.T, G * V, dtype=torch.float32, device=a.device)
-            else:
-                vin, lam = ctx.shared[self.value_mix[1]], self.value_mix[2]
-                assert vin.shape[1] == G * V, "mixed values must have this layer's shape"
-        so.qkv_prep_append(a, 0, self.k_lo, self.v_lo, H, G, D, V, self.q_norm, self.k_norm, ctx.eps, self.freq, self.rot_dims, self.layout,
-                           self.mag, lam, vin, vout, ktable, vtable, ctx.tok_slot, ctx.tok_pos, maps=self.maps)
-        gate = a[:, self.g_lo:] if self.head_gate else None
+        assert out is None or (self.talk is None and self.differential is None)
+        q, gate = a, a[:, self.g_lo:] if self.head_gate else None
+        if self.out_gain is not None:
+            gate = self.out_gain.expand(ctx.T, H)
+        if self.taps:
+            one_row = ctx.max_count == 1
+            q = so.qkv_conv_prep_append(a, self.conv, self.tails[run], one_row, H, G, D, V, self.q_norm, self.k_norm, ctx.eps, self.freq, self.rot_dims,
+                                        self.layout, self.mag, ktable, vtable, ctx.tok_slot, ctx.tok_pos, ctx.tok_off)
+            if self.taps > 1 and not one_row:
+                so.conv_tail_update(self.tails[run], a[:, : self.g_lo], self.taps, ctx.ent_slot, ctx.ent_row0, ctx.ent_count)
+        else:
+            self._prep(ctx, a, ktable, vtable)
         if self.talk is not None and ctx.math == so.MATH_BF16 and self.talk_mc and ctx.max_count >= so.TALK_MC_MIN_ROWS:
             o = so.talk_attn_mc(a, ktable, vtable, ctx.tok_pos, ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count, H, G, D, V, self.scale,
                                 self.talk32, temp=self.head_temp, gate=a[:, self.g_lo:] if self.elem_gate else None, window=self.window,
                                 out=ctx.act_buffer(H * V))
-            return so.linear(o, self.o, self.o_b, math=ctx.math)
+            return o
         if self.talk is not None:
             o = so.talk_attn(a, ktable, vtable, ctx.tok_slot, ctx.tok_pos, ctx.max_pos, H, G, D, V, self.scale, self.talk, temp=self.head_temp,
                              gate=a[:, self.g_lo:] if self.elem_gate else None, window=self.window, out=ctx.act_buffer(H * V))
-            return so.linear(o, self.o, self.o_b, math=ctx.math)
+            return o
         if ctx.math == so.MATH_BF16 and self.mc:
-            o = so.gqa_attn_mc(a, ktable, vtable, ctx.tok_pos, ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count, ctx.max_pos,
-                               H, G, D, V, self.scale, self.sink, self.sink_mode, self.softcap, gate, maps=self.maps, window=self.window,
+            o = so.gqa_attn_mc(q, ktable, vtable, ctx.tok_pos, ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count, ctx.max_pos,
+                               H, G, D, V, self.scale, self.sink, self.sink_mode, self.softcap, gate, out=out, maps=self.maps, window=self.window,
                                keep_first=self.keep_first,
                                diff=(*self.differential, ctx.eps, ctx.act_buffer(H * V)) if self.differential is not None else None)
         else:
-            o = so.gqa_attn(a, ktable, vtable, ctx.tok_slot, ctx.tok_pos, H, G, D, V, self.scale, self.sink, self.sink_mode,
-                            self.softcap, gate, maps=self.maps, window=self.window, keep_first=self.keep_first)
+            o = so.gqa_attn(q, ktable, vtable, ctx.tok_slot, ctx.tok_pos, H, G, D, V, self.scale, self.sink, self.sink_mode,
+                            self.softcap, gate, out=out, maps=self.maps, window=self.window, keep_first=self.keep_first)
             if self.differential is not None:
                 o = so.maps_diff_norm(o, self.differential[0], self.differential[1], ctx.eps, H, V, out=ctx.act_buffer(H * V))
-        return so.linear(o, self.o, self.o_b, math=ctx.math)
+        return o
+
+    def _prep(self, ctx, a, ktable, vtable):
+        """norm and rotation of queries and keys, value mixing, append to the pages"""
+        vin = vout = None
+        lam = 0.0
+        if self.value_mix is not None:
+            if self.value_mix[0] == "source":
+                vout = ctx.shared[self.value_mix[1]] = torch.empty(ctx.T, self.G * self.V, dtype=torch.float32, device=a.device)
+            else:
+                vin, lam = ctx.shared[self.value_mix[1]], self.value_mix[2]
+                assert vin.shape[1] == self.G * self.V, "mixed values must have this layer's shape"
+        so.qkv_prep_append(a, 0, self.k_lo, self.v_lo, self.H, self.G, self.D, self.V, self.q_norm, self.k_norm, ctx.eps, self.freq, self.rot_dims,
+                           self.layout, self.mag, lam, vin, vout, ktable, vtable, ctx.tok_slot, ctx.tok_pos, maps=self.maps)
 
 
 class GatedLinearAttention:
@@ -335,36 +407,101 @@ class GatedLinearAttention:
         return so.linear(on, self.o, math=ctx.math)
 
 
-class StateSpaceMixer:
-    def __init__(self, key, heads, vdim, n_state, groups, taps, norm_groups, w, state):
-        """w: in [2*inner + 2*groups*n_state + heads, width] laid out [z | x | B | C | dt] (inner = heads*vdim), conv [inner +
-        2*groups*n_state, taps] + conv.b over [x | B | C], dt_bias / A_log / D [heads], norm [inner], o [width, inner].
-        Per head (head h reads group h / (heads / groups)):  step = softplus(dt + dt_bias);  S <- exp(-exp(A_log) step) S + step B x^T;
-        y = S^T C + D x;  out = o . (rms-norm over norm_groups parts of (y * silu(z)) * norm)."""
-        assert heads % groups == 0 and (heads * vdim) % norm_groups == 0
-        self.H, self.P, self.N, self.G, self.taps, self.norm_groups = heads, vdim, n_state, groups, int(taps), int(norm_groups)
-        self.inner, self.ch = heads * vdim, heads * vdim + 2 * groups * n_state
-        self.w_in = w["in"].contiguous()
-        assert self.w_in.shape[0] == self.inner + self.ch + heads and w["conv"].shape == (self.ch, self.taps)
-        self.conv, self.conv_b = w["conv"].contiguous(), w["conv.b"].contiguous()
-        self.dt_bias, self.a_log, self.skip = w["dt_bias"].contiguous(), w["A_log"].contiguous(), w["D"].contiguous()
-        self.norm, self.o = w["norm"].contiguous(), w["o"].contiguous()
-        assert self.norm.shape[0] == self.inner and self.o.shape[1] == self.inner
-        self.S = state.add_state(key + ".S", (heads, n_state, vdim))
-        self.tail = state.add_state(key + ".tail", (self.taps - 1, self.ch)) if self.taps > 1 else None
+class Retention:
+    def __init__(self, key, heads, dim, vdim, decay, w, state, rot_dims=0, rot_base=10000.0, rot_layout="halves", rot_scaling=None, runs=1):
+        """w: q / k [heads*dim, width], v / g [heads*vdim, width], o [width, heads*vdim]; decay: one number per head.
+        S <- decay S + (dim^-1/2 k) v^T, o = S^T q, every head over its root mean square, times silu(g h)."""
+        self.H, self.D, self.V, self.k_scale = heads, dim, vdim, dim ** -0.5
+        dev = w["q"].device
+        assert w["q"].shape[0] == w["k"].shape[0] == heads * dim and w["v"].shape[0] == w["g"].shape[0] == w["o"].shape[1] == heads * vdim
+        assert len(decay) == heads and all(0.0 <= float(d) <= 1.0 for d in decay)
+        self.w_in, (self.q_lo, self.k_lo, self.v_lo, self.g_lo) = padded_rows([w["q"], w["k"], w["v"], w["g"]])
+        self.act_cols = (self.g_lo, self.g_lo + heads * vdim)
+        self.o = w["o"].contiguous()
+        logs = torch.tensor([float(d) for d in decay], dtype=torch.float64).log().clamp(min=-1e4)      # (a decay of 0: nothing survives a row)
+        self.log_decay = logs.to(dev)
+        self.rot_dims, self.layout, self.freq = int(rot_dims or 0), so.ROTARY_LAYOUTS[rot_layout], None
+        assert self.rot_dims % 2 == 0 and self.rot_dims <= dim
+        if self.rot_dims:
+            f, mag = rotary_frequencies(self.rot_dims, rot_base, rot_scaling)
+            assert mag == 1.0
+            self.freq = f.to(dev)
+        self.S = [state.add_state(n + ".S", (heads, dim, vdim)) for n in run_names(key, runs)]
 
-    def __call__(self, ctx, h, h16=None):
-        inner, ch, GN = self.inner, self.ch, self.G * self.N
-        a = so.linear(h16 if h16 is not None else h, self.w_in, math=ctx.math)                    # [z | x B C | dt], f32
-        z, xbc, dtr = a[:, :inner], a[:, inner: inner + ch], a[:, inner + ch:]
-        u = so.causal_conv_state(xbc, self.conv, self.conv_b, self.tail, ctx.tok_slot, ctx.tok_off, act="silu")
-        if self.tail is not None:
-            so.conv_tail_update(self.tail, xbc, self.taps, ctx.ent_slot, ctx.ent_row0, ctx.ent_count)
-        y = so.ssd(u, u[:, inner: inner + GN], u[:, inner + GN:], dtr, self.dt_bias, self.a_log, self.S, ctx.ent_slot, ctx.ent_row0,
-                   ctx.ent_count, ctx.max_count, self.H, self.G, self.N, self.P)
-        yn = so.gate_group_rmsnorm(y, z, self.norm, ctx.eps, self.H, self.P, self.norm_groups, x=u, skip=self.skip,
-                                   out=ctx.act_buffer(inner))
-        return so.linear(yn, self.o, math=ctx.math)
+    def __call__(self, ctx, h, h16=None, run=0):
+        a = so.linear(h16 if h16 is not None else h, self.w_in, act="silu", act_cols=self.act_cols, math=ctx.math)       # [q | k | v | silu g]
+        return so.linear(self.mix(ctx, a, run), self.o, math=ctx.math)
+
+    def mix(self, ctx, a, run=0, out=None):
+        H, D, V = self.H, self.D, self.V
+        o = so.retention(a, self.q_lo, self.k_lo, self.v_lo, self.k_scale, self.log_decay, self.freq, self.rot_dims, self.layout, self.S[run], ctx.tok_pos,
+                         ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count, H, D, V)
+        return so.head_rmsnorm_mul(o, None, ctx.eps, H, V, mul=a[:, self.g_lo:], out=out if out is not None else ctx.act_buffer(H * V))
+
+
+class MatrixMemory:
+    def __init__(self, key, heads, dim, vdim, gate_cap, w, state, runs=1, out_scale=1.0):
+        """w: q / k [heads*dim, width], v / g [heads*vdim, width], i / f [heads, width] + i.b / f.b, norm [heads*vdim], o [width, heads*vdim].
+        The recurrence is that of seq_ops.matrix_memory; then every head over its root mean square, times norm, times sigmoid(g h).
+        out_scale: a constant on what the output product reads."""
+        self.H, self.D, self.V, self.cap, self.out_scale = heads, dim, vdim, float(gate_cap), float(out_scale)
+        assert w["q"].shape[0] == w["k"].shape[0] == heads * dim and w["v"].shape[0] == w["g"].shape[0] == w["o"].shape[1] == heads * vdim
+        names = ("q", "k", "v", "g", "i", "f")
+        self.w_in, lo = padded_rows([w[n] for n in names])
+        self.q_lo, self.k_lo, self.v_lo, self.g_lo, self.i_lo, self.f_lo = lo
+        zero = lambda n: torch.zeros(n, dtype=self.w_in.dtype, device=self.w_in.device)
+        self.b_in, _ = padded_rows([w.get(n + ".b", zero(w[n].shape[0])) for n in names])
+        self.act_cols = (self.g_lo, self.g_lo + heads * vdim)
+        self.norm, self.o, self.o_b = w["norm"].contiguous(), w["o"].contiguous(), w.get("o.b")
+        assert self.norm.shape == (heads * vdim,)
+        self.states = [(state.add_state(n + ".S", (heads, dim, vdim)), state.add_state(n + ".n", (heads, dim)),
+                        state.add_state(n + ".m", (heads, so.memory_copies(vdim)))) for n in run_names(key, runs)]
+
+    def __call__(self, ctx, h, h16=None, run=0):
+        a = so.linear(h16 if h16 is not None else h, self.w_in, self.b_in, act="sigmoid", act_cols=self.act_cols, math=ctx.math)
+        return so.linear(self.mix(ctx, a, run), self.o, self.o_b, math=ctx.math)
+
+    def mix(self, ctx, a, run=0, out=None):
+        H, D, V = self.H, self.D, self.V
+        o, den = so.matrix_memory(a[:, self.q_lo:], a[:, self.k_lo:], a[:, self.v_lo:], a[:, self.i_lo:], a[:, self.f_lo:], self.cap, D ** -0.5,
+                                  *self.states[run], ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count, H, D, V)
+        return so.head_rmsnorm_mul(o, self.norm, ctx.eps, H, V, mul=a[:, self.g_lo:], div=den, out_scale=self.out_scale,
+                                   out=out if out is not None else ctx.act_buffer(H * V))
+
+
+class WeightedPair:
+    """Two mixers that read the same input, added with the constants they were built with (out_scale): their input products run as one, and
+    so do their output products -- the sum over both mixers' heads.  A mixer here has w_in / b_in, act_cols (sigmoid columns of its input
+    product, or None), o / o_b, out_scale and mix(ctx, input rows, run, out)."""
+
+    def __init__(self, left, right):
+        self.left, self.right = left, right
+        self.w_in, (_, self.r_lo) = padded_rows([left.w_in, right.w_in])
+        self.b_in = None
+        if left.b_in is not None or right.b_in is not None:
+            zero = lambda m: torch.zeros(m.w_in.shape[0], dtype=self.w_in.dtype, device=self.w_in.device)
+            self.b_in, _ = padded_rows([m.b_in if m.b_in is not None else zero(m) for m in (left, right)])
+        if left.act_cols is not None and right.act_cols is not None:
+            raise ValueError("one activated range of columns per input product")
+        self.act_cols = left.act_cols if right.act_cols is None else tuple(c + self.r_lo for c in right.act_cols)
+        self.k_left = left.o.shape[1]
+        self.o = torch.cat([left.o, right.o], 1).contiguous()
+        biases = [m.o_b.float() * m.out_scale for m in (left, right) if m.o_b is not None]
+        self.bias = sum(biases[1:], biases[0]).contiguous() if biases else None      # f32 [width], scaled
+
+    def rows(self, ctx, h, h16=None, run=0):
+        """-> the output product's rows without `bias`, which a residual step adds (seq_ops.residual_rmsnorm)"""
+        a = so.linear(h16 if h16 is not None else h, self.w_in, self.b_in, act="sigmoid" if self.act_cols else None, act_cols=self.act_cols, math=ctx.math)
+        both = torch.empty(ctx.T, self.o.shape[1], dtype=torch.float32, device=a.device)
+        self.left.mix(ctx, a[:, : self.r_lo], run, out=both[:, : self.k_left])
+        self.right.mix(ctx, a[:, self.r_lo:], run, out=both[:, self.k_left:])
+        return so.linear(both, self.o, math=ctx.math)
+
+    def __call__(self, ctx, h, h16=None, run=0):
+        y = self.rows(ctx, h, h16, run)
+        if self.bias is not None:
+            so.residual_rmsnorm(y, bias=self.bias, x_out=y)
+        return y
 
 
 class SideBySide:
@@ -406,7 +543,7 @@ class GatedMlp:
 
 class ExpertMlp:
     def __init__(self, router, router_b, gates, ups, downs, top, limit=0.0, unit="clamped", scoring="chosen_softmax", correction=None,
-                 identity=0, shared=None, groups=None, group_score="max", renorm=True, factor=1.0):
+                 identity=0, shared=None, groups=None, group_score="max", renorm=True, factor=1.0, shared_gate=None):
         """gates / ups [ff, width] and downs [width, ff] per expert.  unit "clamped": an expert is
         down(glu(min(gate h, limit), clamp(up h, +-limit))); "silu": down(silu(gate h) * (up h)); gates None: unit names an elementwise
         activation, down(act(up h)).
@@ -416,7 +553,9 @@ class ExpertMlp:
         shared: a feed-forward (GatedMlp) that runs for every token and is added, or None.
         groups: None or (count, keep): the router outputs form `count` equal groups of neighbours, a group counts by its largest score
         (logit), or with group_score "top2" by the sum of its two largest choice scores, and only experts of the `keep` best groups can
-        be chosen."""
+        be chosen.
+        shared_gate [1, width]: the shared expert (a clamped GatedMlp) is multiplied by its sigmoid, one number per token; its gate and up
+        rows then join the router's product."""
         self.groups = (int(groups[0]), int(groups[1])) if groups else (1, 1)
         self.E, self.top, self.limit = len(ups), int(top), float(limit)
         self.unit = {"clamped": so.UNIT_CLAMPED, "silu": so.UNIT_SILU}[unit] if gates is not None else None
@@ -432,12 +571,47 @@ class ExpertMlp:
         assert self.router.shape[0] == self.E + self.identity and 0 < self.top <= self.E + self.identity
         assert self.correction is None or (self.scoring != so.ROUTE_CHOSEN_SOFTMAX and self.correction.shape == (self.E + self.identity,))
 
+        self.w_x = None
+        if shared_gate is not None:
+            assert shared is not None and shared.limit is not None and self.identity == 0
+            n = self.router.shape[0]
+            zero = lambda k: torch.zeros(k, dtype=self.router.dtype, device=self.router.device)
+            self.w_x, (_, self.sg_lo, self.gu_lo) = padded_rows([self.router, shared_gate, shared.w_gu])
+            if self.router_b is not None:
+                self.b_x, _ = padded_rows([self.router_b, zero(1), zero(shared.w_gu.shape[0])])
+            else:
+                self.b_x = None
+
+    def parts(self, ctx, h, h16=None):
+        """-> ((rows, dst, wts), the gated shared expert's rows or None): what the residual step sums (seq_ops.residual_rmsnorm).  Router,
+        shared gate and the shared expert's first product are ONE product: its sums are f32 either way."""
+        x = h16 if h16 is not None else h
+        if self.w_x is None:
+            assert self.shared is None and not self.identity
+            return self.__call__(ctx, h, h16, defer=True), None
+        z = so.linear(x, self.w_x, self.b_x, act="sigmoid", act_cols=(self.sg_lo, self.sg_lo + 1), math=ctx.math)
+        routed = self._routed(ctx, x, z[:, : self.router.shape[0]])
+        F = self.shared.F
+        g = so.moe_glu(z[:, self.gu_lo:], F, self.shared.limit, GLU_SLOPE, ctx.act_buffer(F))
+        return routed[1:], so.linear(g, self.shared.down, mul=z[:, self.sg_lo: self.sg_lo + 1], mul_group=True, math=ctx.math)
+
     def __call__(self, ctx, h, h16=None, defer=False):
         """defer: where the result is nothing but the weighted sum of routed rows, (rows, dst, wts) is returned instead, to be summed
         inside the residual step (seq_ops.residual_layernorm)"""
         x = h16 if h16 is not None else h
-        T, R = ctx.T, ctx.T * self.top
+        if self.w_x is not None:
+            (d, dst, wts), add = self.parts(ctx, h, h16)
+            return so.moe_combine(d, dst, wts, ctx.T, self.top, add=add)
         logits = so.linear(x, self.router, self.router_b, math=so.MATH_F32 if ctx.math == so.MATH_F32 else so.MATH_F32_STREAM)
+        ids, d, dst, wts = self._routed(ctx, x, logits)
+        if defer and not self.identity and self.shared is None:
+            return d, dst, wts
+        add = self.shared(ctx, h, h16) if self.shared is not None else None
+        return so.moe_combine(d, dst, wts, ctx.T, self.top, ids=ids if self.identity else None, n_real=self.E, own=x, add=add)
+
+    def _routed(self, ctx, x, logits):
+        """-> (chosen ids, the experts' output rows grouped by expert, where each (token, choice) went, weights)"""
+        T, R = ctx.T, ctx.T * self.top
         ids, wts, seg, src_row, dst = so.moe_route(logits, self.top, self.scoring, self.correction, self.groups, **self.rule)
         # the pairs of the identity experts sort behind those of the real ones: the expert products never see their rows
         if self.act is not None:
@@ -445,11 +619,7 @@ class ExpertMlp:
         else:
             gu = so.linear_segmented(x, self.w_up, seg, src_row, T, R, math=ctx.math)
             y = so.moe_glu(gu, self.F, self.limit, GLU_SLOPE, ctx_rows(ctx, R, self.F), unit=self.unit)
-        d = so.linear_segmented(y, self.w_down, seg, None, T, R, math=ctx.math)
-        if defer and not self.identity and self.shared is None:
-            return d, dst, wts
-        add = self.shared(ctx, h, h16) if self.shared is not None else None
-        return so.moe_combine(d, dst, wts, T, self.top, ids=ids if self.identity else None, n_real=self.E, own=x, add=add)
+        return ids, so.linear_segmented(y, self.w_down, seg, None, T, R, math=ctx.math), dst, wts
 
 
 def ctx_rows(ctx, rows, n):

@@ -47,5 +47,18 @@ def read_config(path):
         return json.load(f)
 
 
+def layer_runs(n_layers, loop):
+    """[(layer, which run of that layer, pass that starts here or None)] in the order the layers run"""
+    if not loop:
+        return [(i, 0, None) for i in range(n_layers)]
+    a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
+    if not 0 <= a < b <= n_layers or times < 1:
+        raise ValueError(f"loop {loop!r} does not fit {n_layers} layers")
+    runs = [(i, 0, None) for i in range(a)]
+    for t in range(times):
+        runs += [(i, t, t if i == a else None) for i in range(a, b)]
+    return runs + [(i, 0, None) for i in range(b, n_layers)]
+
+
 def _load_builtin():
-    from . import filipel, modanex, qwen2, tobilorn, vabanex, vogusun  # noqa: F401  (registration on import)
+    from . import filipel, modanex, qwen2, tobilorn, vabanex, vogusun, zusuvik  # noqa: F401  (registration on import)

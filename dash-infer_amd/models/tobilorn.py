@@ -23,24 +23,11 @@ import torch
 
 from .. import mixers
 from .. import seq_ops as so
-from . import register
+from . import layer_runs, register
 
 
 def _sub(tensors, prefix):
     return {k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)}
-
-
-def layer_runs(n_layers, loop):
-    """[(layer, which run of that layer, pass that starts here or None)] in the order the layers run"""
-    if not loop:
-        return [(i, 0, None) for i in range(n_layers)]
-    a, b, times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
-    if not 0 <= a < b <= n_layers or times < 1:
-        raise ValueError(f"loop {loop!r} does not fit {n_layers} layers")
-    runs = [(i, 0, None) for i in range(a)]
-    for t in range(times):
-        runs += [(i, t, t if i == a else None) for i in range(a, b)]
-    return runs + [(i, 0, None) for i in range(b, n_layers)]
 
 
 class _Layer:

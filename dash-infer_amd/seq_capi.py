@@ -49,7 +49,15 @@ _SIGS = {
                                 i32, f32, i32, i32, i32, i32, vp, sz, vp, i32, lng, f32, f32, f32]),
     "dihip_gla_workspace_bytes": (sz, [i32, i32, i32, i32, i32, i32, i32]),
     "dihip_gla": (i32, [vp, vp, lng, vp, lng, vp, lng, vp, lng, vp, lng, f32, f32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, vp, sz]),
-    "dihip_head_rmsnorm_mul": (i32, [vp, vp, i32, lng, vp, lng, vp, i32, f32, vp, lng, i32, i32, i32]),
+    "dihip_head_rmsnorm_mul": (i32, [vp, vp, i32, lng, vp, lng, vp, i32, i32, f32, vp, vp, lng, f32, i32, i32, i32]),
+    "dihip_decay_attn_workspace_bytes": (sz, [i32, i32, i32, i32, i32, i32, i32, i32]),
+    "dihip_retention": (i32, [vp, vp, lng, vp, lng, i32, i32, i32, f32, vp, vp, i32, i32, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, vp, sz]),
+    "dihip_matrix_memory": (i32, [vp, vp, lng, vp, vp, lng, vp, lng, vp, lng, vp, vp, lng, f32, f32, vp, vp, vp, i32, vp, vp, vp, i32, i32, i32, i32, i32,
+                                  i32, i32, vp, sz]),
+    "dihip_qkv_conv_prep_append": (i32, [vp, vp, lng, vp, i32, vp, i32, i32, i32, i32, i32, vp, vp, i32, f32, vp, i32, i32, f32, vp, lng, vp, vp, i32, i32,
+                                         i32, vp, vp, vp, i32]),
+    "dihip_residual_rmsnorm": (i32, [vp, vp, vp, vp, lng, vp, lng, vp, vp, lng, vp, lng, vp, vp, i32, vp, vp, vp, i32, f32, f32, f32, vp, vp, i32, lng, i32,
+                                     i32]),
     "dihip_seq_moe_route": (i32, [vp, vp, lng, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, vp, i32, i32, i32, i32, i32, f32]),
     "dihip_seq_moe_glu": (i32, [vp, vp, i32, lng, vp, lng, i32, i32, f32, f32, i32]),
     "dihip_seq_moe_combine": (i32, [vp, vp, lng, vp, lng, vp, vp, i32, i32, i32, vp, i32, vp, i32, lng, vp, lng]),

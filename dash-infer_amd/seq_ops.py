@@ -248,6 +248,23 @@ def qkv_prep_append(a, q_off, k_off, v_off, H, G, D, DV, qnorm, knorm, eps, freq
           "dihip_qkv_prep_append")
 
 
+def qkv_conv_prep_append(x, conv, tail, one_row, H, G, D, DV, qnorm, knorm, eps, freq, rot_dims, layout, mag, ktable, vtable, tok_slot, tok_pos, tok_off):
+    """short convolution on every channel of x = [q | k | v] (f32 rows), norms over the whole query / key row, rotation, append of k and v to
+    their pages; one_row: every portion of the step has one row (its tail moves on here) -> the queries, f32 [T, H * D]"""
+    T, taps = x.shape[0], conv.shape[1]
+    C = (H + G) * D + G * DV
+    assert x.dtype == torch.float32 and x.shape[1] >= C and conv.shape == (C, taps) and conv.is_contiguous() and ktable.dtype == vtable.dtype
+    assert ktable.row_elems == G * D and vtable.row_elems == G * DV and (taps == 1 or (tail.shape[1:] == (taps - 1, C) and tail.is_contiguous()))
+    assert (qnorm is None or qnorm.shape == (H * D,)) and (knorm is None or knorm.shape == (G * D,))
+    assert all(w is None or w.dtype == conv.dtype for w in (qnorm, knorm))
+    q = torch.empty(T, H * D, dtype=torch.float32, device=x.device)
+    check(lib().dihip_qkv_conv_prep_append(stream(), ptr(x), _rows(x), ptr(conv), taps, ptr(tail), 1 if one_row else 0, H, G, D, DV, ptr(qnorm), ptr(knorm),
+                                           dt(conv), float(eps), ptr(freq), int(rot_dims), int(layout), float(mag), ptr(q), _rows(q), ptr(ktable.ptrs),
+                                           ptr(vtable.ptrs), ktable.max_spans, ktable.span_len, _DT[ktable.dtype], ptr(tok_slot), ptr(tok_pos),
+                                           ptr(tok_off), T), "dihip_qkv_conv_prep_append")
+    return q
+
+
 ROTARY_LAYOUTS = {"pairs": 0, "halves": 1}      # dimension 2i turns with 2i + 1 / dimension i with i + half
 SINK_NONE, SINK_PER_HEAD, SINK_ZERO = 0, 1, 2
 
@@ -322,12 +339,64 @@ def gla(q, k, v, z, q_scale, tau, state, ent_slot, ent_row0, ent_count, max_coun
     return o
 
 
-def head_rmsnorm_mul(x, gamma, eps, H, DV, mul=None, out=None):
+def head_rmsnorm_mul(x, gamma, eps, H, DV, mul=None, out=None, div=None, out_scale=1.0):
+    """per head: v = x * div[t, h]; v / rms(v) * gamma * mul * out_scale; gamma [DV] shared by the heads, [H * DV], or None"""
     T = x.shape[0]
     y = out if out is not None else torch.empty(T, H * DV, dtype=torch.float32, device=x.device)
-    check(lib().dihip_head_rmsnorm_mul(stream(), ptr(y), dt(y), _rows(y), ptr(x), _rows(x), ptr(gamma), dt(gamma), float(eps), ptr(mul),
-                                       _rows(mul) if mul is not None else 0, T, H, DV), "dihip_head_rmsnorm_mul")
+    assert gamma is None or gamma.numel() in (DV, H * DV)
+    assert div is None or (div.shape == (T, H) and div.is_contiguous() and div.dtype == torch.float32)
+    check(lib().dihip_head_rmsnorm_mul(stream(), ptr(y), dt(y), _rows(y), ptr(x), _rows(x), ptr(gamma), 1 if gamma is not None and gamma.numel() != DV else 0,
+                                       dt(gamma) if gamma is not None else F32_CODE, float(eps), ptr(div), ptr(mul), _rows(mul) if mul is not None else 0,
+                                       float(out_scale), T, H, DV), "dihip_head_rmsnorm_mul")
     return y
+
+
+CHUNKED_DECAY_ROWS = 32   # portions from this length on run as chunks side by side
+
+
+def _decay_workspace(T, E, max_count, H, D, DV, gated, chunked, device):
+    if chunked is None:
+        chunked = max_count >= CHUNKED_DECAY_ROWS
+    n = int(lib().dihip_decay_attn_workspace_bytes(T, E, int(max_count), H, D, DV, gated, 1 if chunked else 0))
+    return 1 if chunked else 0, torch.empty(max(n, 16), dtype=torch.uint8, device=device)
+
+
+def retention(rows, q_off, k_off, v_off, k_scale, log_decay, freq, rot_dims, layout, state, tok_pos, ent_slot, ent_row0, ent_count, max_count, H, D,
+              DV, out=None, chunked=None):
+    """rows f32 [T, .] hold q, k [H, D] and v [H, DV] at their offsets (q and k may be rotated in place); log_decay f64 [H]; state
+    [slots, H, D, DV] f32 -> f32 [T, H * DV]"""
+    T, E = rows.shape[0], ent_slot.shape[0]
+    assert state.shape[1:] == (H, D, DV) and state.is_contiguous() and log_decay.dtype == torch.float64 and log_decay.shape == (H,)
+    assert rows.dtype == torch.float32 and rows.shape[1] >= max(q_off + H * D, k_off + H * D, v_off + H * DV) and (not rot_dims or freq.shape[0] >= rot_dims // 2)
+    o = out if out is not None else torch.empty(T, H * DV, dtype=torch.float32, device=rows.device)
+    chunked, ws = _decay_workspace(T, E, max_count, H, D, DV, 0, chunked, rows.device)
+    check(lib().dihip_retention(stream(), ptr(o), _rows(o), ptr(rows), _rows(rows), int(q_off), int(k_off), int(v_off), float(k_scale), ptr(log_decay),
+                                ptr(freq), int(rot_dims), int(layout), ptr(state), ptr(tok_pos), ptr(ent_slot), ptr(ent_row0), ptr(ent_count), T, E,
+                                int(max_count), int(H), int(D), int(DV), chunked, ptr(ws), ws.numel()), "dihip_retention")
+    return o
+
+
+def memory_copies(DV):
+    """copies of the running maximum the matrix memory keeps: one per 64 value columns"""
+    return (DV + 63) // 64
+
+
+def matrix_memory(q, k, v, gate_i, gate_f, cap, q_scale, state_s, state_n, state_m, ent_slot, ent_row0, ent_count, max_count, H, D, DV, out=None,
+                  chunked=None):
+    """q, k f32 [T, >= H * D], v [T, >= H * DV], raw gates [T, >= H] rows; state_s [slots, H, D, DV], state_n [slots, H, D], state_m
+    [slots, H, memory_copies(DV)] -> (out f32 [T, H * DV], den f32 [T, H]): the result is out * den"""
+    T, E = q.shape[0], ent_slot.shape[0]
+    assert state_s.shape[1:] == (H, D, DV) and state_n.shape[1:] == (H, D) and state_m.shape[1:] == (H, memory_copies(DV))
+    assert all(t.is_contiguous() for t in (state_s, state_n, state_m)) and _rows(gate_i) == _rows(gate_f)
+    assert q.shape[1] >= H * D and k.shape[1] >= H * D and v.shape[1] >= H * DV and gate_i.shape[1] >= H and gate_f.shape[1] >= H
+    o = out if out is not None else torch.empty(T, H * DV, dtype=torch.float32, device=q.device)
+    den = torch.empty(T, H, dtype=torch.float32, device=q.device)
+    chunked, ws = _decay_workspace(T, E, max_count, H, D, DV, 1, chunked, q.device)
+    check(lib().dihip_matrix_memory(stream(), ptr(o), _rows(o), ptr(den), ptr(q), _rows(q), ptr(k), _rows(k), ptr(v), _rows(v), ptr(gate_i), ptr(gate_f),
+                                    _rows(gate_i), float(cap), float(q_scale), ptr(state_s), ptr(state_n), ptr(state_m), state_m.shape[2], ptr(ent_slot),
+                                    ptr(ent_row0), ptr(ent_count), T, E, int(max_count), int(H), int(D), int(DV), chunked, ptr(ws), ws.numel()),
+          "dihip_matrix_memory")
+    return o, den
 
 
 # scores: the logits (weights = softmax over the chosen ones) / softmax over all logits / the sigmoid of each logit
@@ -388,6 +457,28 @@ def residual_layernorm(x_in, w=None, a=None, b=None, mult=1.0, eps=1e-5, x_out=N
                                          dt(w) if w is not None else F32_CODE, float(eps), ptr(h), dt(h) if h is not None else F32_CODE,
                                          _rows(h) if h is not None else 0, M, K), "dihip_residual_layernorm")
     return h
+
+
+def residual_rmsnorm(x_in, w1=None, w2=None, a=None, b=None, bias=None, again=None, routed=None, add=1.0, scale=1.0, eps=1e-5, x_out=None,
+                     row_idx=None, out_dtype=torch.float32):
+    """x_out = x_in + (a + b + bias + the routed rows' weighted sum) + again;  h1, h2 = x_out / rms(x_out) * (add + w1 / w2) * scale -> (h1, h2)
+    (None where the weight is None).  bias f32 [K]; routed as residual_layernorm takes it; row_idx: the norm of the chosen rows alone."""
+    K = x_in.shape[1]
+    M = x_in.shape[0] if row_idx is None else row_idx.shape[0]
+    assert x_in.is_contiguous() and x_in.dtype == torch.float32 and (x_out is None or x_out.is_contiguous())
+    rows, dst, wts = routed if routed is not None else (None, None, None)
+    assert routed is None or (rows.dtype == wts.dtype == torch.float32 and rows.shape[1] == K and wts.shape[0] == M and wts.is_contiguous())
+    assert all(y is None or (y.dtype == torch.float32 and y.shape == (M, K)) for y in (a, b, again)) and (bias is None or (bias.dtype == torch.float32 and bias.shape == (K,)))
+    assert w1 is None or w2 is None or w1.dtype == w2.dtype
+    h1 = torch.empty(M, K, dtype=out_dtype, device=x_in.device) if w1 is not None else None
+    h2 = torch.empty(M, K, dtype=out_dtype, device=x_in.device) if w2 is not None else None
+    w, h = (w1 if w1 is not None else w2), (h1 if h1 is not None else h2)
+    check(lib().dihip_residual_rmsnorm(stream(), ptr(x_out), ptr(x_in), ptr(a), _rows(a) if a is not None else 0, ptr(b), _rows(b) if b is not None else 0,
+                                       ptr(bias), ptr(again), _rows(again) if again is not None else 0, ptr(rows), _rows(rows) if rows is not None else 0,
+                                       ptr(dst), ptr(wts), wts.shape[1] if wts is not None else 0, ptr(row_idx), ptr(w1), ptr(w2),
+                                       dt(w) if w is not None else F32_CODE, float(add), float(scale), float(eps), ptr(h1), ptr(h2),
+                                       dt(h) if h is not None else F32_CODE, _rows(h) if h is not None else 0, M, K), "dihip_residual_rmsnorm")
+    return h1, h2
 
 
 def polynorm(z, coef, eps, out):

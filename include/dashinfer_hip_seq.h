@@ -68,6 +68,14 @@ int dihip_add_dyt(void* stream, float* x_out, const float* x_in, const float* a,
 int dihip_residual_layernorm(void* stream, float* x_out, const float* x_in, const float* a, long lda, const float* b, long ldb,
                              const float* rows, long ldr, const int32_t* dst, const float* wts, int top, float mult, const int32_t* row_idx, const void* w, const void* bias, int w_dtype, float eps, void* h,
                              int h_dtype, long ldh, int M, int K);
+/* The same step with RMS norms, two of them for sublayers that have an input norm each:
+ *   x_out[r] = x_in[r] + (a[r] + b[r] + bias + sum_k wts[r, k] * rows[dst[r * top + k]]) + again[r]     (every part may be NULL; bias f32 [K])
+ *   h1[i], h2[i] = x_out[r] / sqrt(mean(x_out[r]^2) + eps) * (add + w1 / w2) * scale                   (w1 / w2 NULL: not written)
+ * with row_idx: the norm of the chosen rows alone (x_out NULL). */
+int dihip_residual_rmsnorm(void* stream, float* x_out, const float* x_in, const float* a, long lda, const float* b, long ldb, const float* bias,
+                           const float* again, long ldagain, const float* rows, long ldr, const int32_t* dst, const float* wts, int top,
+                           const int32_t* row_idx, const void* w1, const void* w2, int w_dtype, float add, float scale, float eps, void* h1,
+                           void* h2, int h_dtype, long ldh, int M, int K);
 /* y[t] = c0 z / rms(z) + c1 z^2 / rms(z^2) + c2 z^3 / rms(z^3) + c3,  powers per element, rms(v) = sqrt(mean(v^2) + eps) over the
  * F elements of the row; coef = (c0, c1, c2, c3) of w_dtype */
 int dihip_polynorm(void* stream, void* y, int y_dtype, long ldy, const float* z, long ldz, const void* coef, int w_dtype, float eps,
@@ -140,11 +148,21 @@ int dihip_qkv_prep_append(void* stream, float* qkv, long ld, int q_off, int k_of
                           void* const* kspans, void* const* vspans, int span_stride, int span_len, int cache_dtype,
                           const int32_t* tok_slot, const int32_t* tok_pos, int T);
 
+/* step 1 of a layer with short convolutions: per channel c of x[t] = [q [H, D] | k [G, D] | v [G, DV]] (f32)
+ *   u[t, c] = sum_{j < taps} conv[c, j] * x[t - (taps - 1) + j, c]   (earlier steps' inputs: tail, as dihip_causal_conv_state has it),
+ * then the whole query row and the whole key row are divided by their root mean square and scaled by qnorm [H * D] / knorm [G * D]
+ * (NULL: no norm), rotated per head as above; queries go to q_out, keys and values to their pages.  write_tail: every portion of the step
+ * has one row, the tail is moved on here (else: dihip_conv_tail_update afterwards). */
+int dihip_qkv_conv_prep_append(void* stream, const float* x, long ld, const void* conv, int taps, float* tail, int write_tail, int H, int G, int D,
+                               int DV, const void* qnorm, const void* knorm, int w_dtype, float eps, const float* freq, int rot_dims,
+                               int layout, float mag, float* q_out, long ldq, void* const* kspans, void* const* vspans, int span_stride,
+                               int span_len, int cache_dtype, const int32_t* tok_slot, const int32_t* tok_pos, const int32_t* tok_off, int T);
+
 /* step 2: causal attention of every row over its sequence's pages; query head h reads key/value head h / (H / G):
  *   s_j = scale * q[t, h, m] . k_j[m],  softcap > 0: s_j <- softcap * tanh(s_j / softcap),
  *   over the keys j <= p = tok_pos[t] with  p - j < window  or  j < keep_first  (window <= 0: every j <= p)
  *   p = softmax over {s_j} and, with sink_mode 1 / 2, one more logit sink[h] / 0 that has no value
- *   out[t, h, m] = gate[t, h] * sum_j p_j v_j   (gate NULL: 1)
+ *   out[t, h, m] = gate[t, h] * sum_j p_j v_j   (gate NULL: 1; ldg 0: one row [H] for every t)
  * for every map m < maps of the head (each a softmax of its own over the same values).
  * q [T, H, maps, D], out [T, H, maps, DV] f32.  Every product and sum in f32. */
 int dihip_gqa_attn(void* stream, float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
@@ -178,9 +196,30 @@ int dihip_gla(void* stream, float* out, long ldo, const float* q, long ldq, cons
               const float* z, long ldz, float q_scale, float tau, float* state, const int32_t* ent_slot,
               const int32_t* ent_row0, const int32_t* ent_count, int T, int E, int max_count, int H, int D, int DV,
               int chunked, void* ws, size_t ws_bytes);
-/* y[t, h, :] = x[t, h, :] / sqrt(mean(x[t, h, :]^2) + eps) * gamma * mul[t, h, :]   (gamma [DV] shared by the heads; mul NULL: 1) */
-int dihip_head_rmsnorm_mul(void* stream, void* y, int y_dtype, long ldy, const float* x, long ldx, const void* gamma,
-                           int w_dtype, float eps, const float* mul, long ldm, int T, int H, int DV);
+/* v = x[t, h, :] * div[t, h]  (div [T, H]; NULL: x itself);  y[t, h, :] = v / sqrt(mean(v^2) + eps) * gamma * mul[t, h, :] * out_scale
+ * gamma: [DV] shared by the heads, [H * DV] with gamma_per_head, NULL: 1;  mul NULL: 1 */
+int dihip_head_rmsnorm_mul(void* stream, void* y, int y_dtype, long ldy, const float* x, long ldx, const void* gamma, int gamma_per_head,
+                           int w_dtype, float eps, const float* div, const float* mul, long ldm, float out_scale, int T, int H, int DV);
+
+/* Linear attention with one decay per head (f32), S [slots][H][D][DV] carried per slot:  S <- a S + w k v^T,  out[t, h] = S^T q.
+ * chunked != 0: portions cut into chunks of 64 rows that run side by side on the f32 matrix instructions (f32 rounding differs).
+ * workspace (16-byte aligned): .._workspace_bytes, gated = 1 for the matrix memory; none without chunks.  At most 512 key channels.
+ *   retention: rows [q | k | v] at q_off / k_off / v_off ([H, D], [H, D], [H, DV]); q and k rotate on their first rot_dims dimensions (layout
+ *   0: dimension 2i with 2i + 1, 1: i with i + rot_dims / 2; angles tok_pos * freq; the rows may be rotated in place); k times k_scale;
+ *   a = exp(log_decay[h]) (f64 [H]), w = 1.
+ *   matrix memory (xLSTM): log gates i = cap tanh(gate_i / cap), f = logsigmoid(cap tanh(gate_f / cap)); with the running maximum m:
+ *   m' = max(f + m, i), a = exp(f + m - m'), w = exp(i - m'), n <- a n + w k;  q times q_scale;
+ *   den[t, h] = 1 / (max(|n . q|, exp(-m')) + 1e-6) is what out[t, h] is still to be multiplied by.  state_n [slots][H][D], state_m
+ *   [slots][H][m_copies], m_copies = ceil(DV / 64) equal copies. */
+size_t dihip_decay_attn_workspace_bytes(int T, int E, int max_count, int H, int D, int DV, int gated, int chunked);
+int dihip_retention(void* stream, float* out, long ldo, float* rows, long ld, int q_off, int k_off, int v_off, float k_scale,
+                    const double* log_decay, const float* freq, int rot_dims, int layout, float* state, const int32_t* tok_pos,
+                    const int32_t* ent_slot, const int32_t* ent_row0, const int32_t* ent_count, int T, int E, int max_count, int H, int D,
+                    int DV, int chunked, void* ws, size_t ws_bytes);
+int dihip_matrix_memory(void* stream, float* out, long ldo, float* den, const float* q, long ldq, const float* k, long ldk, const float* v,
+                        long ldv, const float* gate_i, const float* gate_f, long ldg, float cap, float q_scale, float* state_s,
+                        float* state_n, float* state_m, int m_copies, const int32_t* ent_slot, const int32_t* ent_row0,
+                        const int32_t* ent_count, int T, int E, int max_count, int H, int D, int DV, int chunked, void* ws, size_t ws_bytes);
 
 /* Mixture of experts, per token: scores s = the E logits (scoring 0), softmax over them (1) or the sigmoid of each (2); the `top`
  * experts of largest choice score s + correction[e] are chosen (ties: the lower index; correction [E] of w_dtype, NULL: none; not

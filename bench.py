@@ -1031,7 +1031,7 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)
-    ap.add_argument("--workload", default="int4_b1", choices=list(WORKLOADS) + ["launch_selftest", "modanex_layers", "vogusun_layers", "tobilorn_layers", "filipel_layers", "vabanex_layers"])  # int4_b1 = the headline configuration
+    ap.add_argument("--workload", default="int4_b1", choices=list(WORKLOADS) + ["launch_selftest", "modanex_layers", "vogusun_layers", "tobilorn_layers", "filipel_layers", "vabanex_layers", "zusuvik_layers"])  # int4_b1 = the headline configuration
     ap.add_argument("--layers", type=int, default=None, help="debug: fewer decoder layers (result marked invalid)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-graph", action="store_true", help="debug: eager launches instead of hipGraph replay")
@@ -1132,6 +1132,16 @@ def main():
         out = vabanex_bench.run(args)
         os.makedirs(os.path.join(ROOT, "gpurun_out"), exist_ok=True)
         with open(os.path.join(ROOT, "gpurun_out", "bench_vabanex_layers.json"), "w") as f:
+            json.dump(out, f, indent=1)
+        print(json.dumps(out), flush=True)
+        return
+    if args.workload == "zusuvik_layers":
+        # the sequence engine on random Zusuvik models of real layer sizes, beside Vogusun models of equal size (dash-infer_amd/zusuvik_bench.py)
+        assert world == 1, "zusuvik_layers is a one-GPU workload"
+        from dash_infer_amd import zusuvik_bench
+        out = zusuvik_bench.run(args)
+        os.makedirs(os.path.join(ROOT, "gpurun_out"), exist_ok=True)
+        with open(os.path.join(ROOT, "gpurun_out", "bench_zusuvik_layers.json"), "w") as f:
             json.dump(out, f, indent=1)
         print(json.dumps(out), flush=True)
         return

@@ -101,12 +101,12 @@ __global__ __launch_bounds__(256) void qkv_prep_append_kernel(PrepArgs a) {
 }
 
 // ------------------------------------------------------------------------------------------------ convolution + prep + append
-// u[c] = sum_j w[c, j] x[t - (taps - 1) + j, c] for the channels [q | k | v] of the rows x (inputs of earlier steps: the slot's tail), then
+// u[c] = sum_j w[j, c] x[t - (taps - 1) + j, c] for the channels [q | k | v] of the rows x (inputs of earlier steps: the slot's tail), then
 // the query row and the key row as a whole are divided by their root mean square and weighted, their heads rotated; queries go to q_out,
 // keys and values to their pages.  A workgroup per (row, q / k / v); the convolved row is kept in LDS.
 struct ConvPrepArgs {
   const float* x; long ld;                     // [T][HD + GD + GV]
-  const void* w; const void* qnorm; const void* knorm; int wdt; int taps;
+  const void* w; const void* qnorm; const void* knorm; int wdt; int taps;      // w: [taps][HD + GD + GV]
   float* tail; int write_tail;                 // [slots][taps - 1][C]; write_tail: every portion has ONE row, which also moves its tail on
   float eps; const float* freq; int rot_dims, pairs; float mag;
   float* q_out; long ldq;
@@ -138,7 +138,7 @@ __global__ __launch_bounds__(NT) void qkv_conv_prep_append_kernel(ConvPrepArgs a
     for (int k = 0; k < a.taps; ++k) {
       const int d = nt - k, o = off - d;
       const float v = o >= 0 ? a.x[(size_t)(t - d) * a.ld + c] : tl[(size_t)(nt + o) * C + c];
-      acc = __builtin_fmaf(ld_any(a.w, (size_t)c * a.taps + k, a.wdt), v, acc);
+      acc = __builtin_fmaf(ld_any(a.w, (size_t)k * C + c, a.wdt), v, acc);
       if (a.write_tail && k > 0) tl[(size_t)(k - 1) * C + c] = v;      // (off == 0: row k - 1 was read in the turn before)
     }
     ss = __builtin_fmaf(acc, acc, ss);
@@ -170,9 +170,138 @@ __global__ __launch_bounds__(NT) void qkv_conv_prep_append_kernel(ConvPrepArgs a
   }
 }
 
+// The same for rows of whole 16-byte units (head sizes that are multiples of 4): a thread owns EPT units of 4 channels, all of its loads are
+// issued before the first use, the convolved row stays in registers; neighbouring dimensions rotate inside a unit, halves through LDS.
+// The number of threads follows the row's length alone: a row's bits do not depend on the batch.
+template <int WT>
+__device__ __forceinline__ f32x4_t load_w4(const void* p, size_t i) {
+  if constexpr (WT == DIHIP_F32) return *reinterpret_cast<const f32x4_t*>((const float*)p + i);
+  const u32x2_t r = *reinterpret_cast<const u32x2_t*>((const uint16_t*)p + i);
+  return f32x4_t{__uint_as_float(r[0] << 16), __uint_as_float(r[0] & 0xffff0000u), __uint_as_float(r[1] << 16), __uint_as_float(r[1] & 0xffff0000u)};
+}
+__device__ __forceinline__ void store4(void* p, size_t i, int dt, const f32x4_t& v) {
+  if (dt == DIHIP_F32) *reinterpret_cast<f32x4_t*>((float*)p + i) = v;
+  else *reinterpret_cast<u32x2_t*>((uint16_t*)p + i) = u32x2_t{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
+}
+
+template <int WT, int NT, int EPT>
+__global__ __launch_bounds__(NT) void qkv_conv_prep_append_vec_kernel(ConvPrepArgs a) {
+  extern __shared__ float us[];                                         // halves: the normed row
+  __shared__ float cs[128], sn[128], red[NT / 64];
+  const int t = blockIdx.x, part = blockIdx.y, tid = threadIdx.x;      // part 0: q, 1: k, 2: v
+  const int nt = a.taps - 1, C = a.HD + a.GD + a.GV, half = a.rot_dims >> 1;
+  const int c0 = part == 0 ? 0 : (part == 1 ? a.HD : a.HD + a.GD), n = part == 0 ? a.HD : (part == 1 ? a.GD : a.GV);
+  if (tid * 4 >= n && tid >= 64 * ((n / 4 + 63) / 64) && part == 2) return;      // (values: no barrier follows; whole waves past the row)
+  const int pos = a.tok_pos[t], off = a.tok_off[t], slot = a.tok_slot[t];
+  float* tl = a.tail ? a.tail + (size_t)slot * nt * C : nullptr;
+  int c[EPT];
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) c[e] = min((tid + e * NT) * 4, n - 4);          // units past the row repeat its last one and are not stored
+  f32x4_t u[EPT], gm[EPT];
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) u[e] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const void* gamma = part == 0 ? a.qnorm : (part == 1 ? a.knorm : nullptr);
+  if (gamma) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) gm[e] = load_w4<WT>(gamma, c[e]);
+  }
+  for (int k0 = 0; k0 < a.taps; k0 += 4) {
+    f32x4_t xv[4][EPT], wv[4][EPT];
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+      const int k = min(k0 + kk, a.taps - 1), d = nt - k, o = off - d;
+      const float* src = o >= 0 ? a.x + (size_t)(t - d) * a.ld + c0 : tl + (size_t)(nt + o) * C + c0;
+#pragma unroll
+      for (int e = 0; e < EPT; ++e) {
+        xv[kk][e] = *reinterpret_cast<const f32x4_t*>(src + c[e]);
+        wv[kk][e] = load_w4<WT>(a.w, (size_t)k * C + c0 + c[e]);
+      }
+    }
+    if (k0 == 0 && part < 2 && tid < half) {       // while the loads are in flight
+      float s_, c_;
+      rope_sincos((uint32_t)pos, a.freq[tid], &s_, &c_);
+      sn[tid] = s_ * a.mag;
+      cs[tid] = c_ * a.mag;
+    }
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+      if (k0 + kk < a.taps) {
+#pragma unroll
+        for (int e = 0; e < EPT; ++e) {
+#pragma unroll
+          for (int x = 0; x < 4; ++x) u[e][x] = __builtin_fmaf(wv[kk][e][x], xv[kk][e][x], u[e][x]);
+          if (a.write_tail && k0 + kk > 0 && (tid + e * NT) * 4 < n)      // tail row k - 1 <- the input of tap k (row k - 1 has been read)
+            *reinterpret_cast<f32x4_t*>(tl + (size_t)(k0 + kk - 1) * C + c0 + c[e]) = xv[kk][e];
+        }
+      }
+    }
+  }
+  const size_t sp = (size_t)slot * a.span_stride + pos / a.span_len, in_span = (size_t)(pos % a.span_len);
+  if (part == 2) {
+    void* vdst = a.vspans[sp];
+#pragma unroll
+    for (int e = 0; e < EPT; ++e)
+      if ((tid + e * NT) * 4 < n) store4(vdst, in_span * n + c[e], a.cdt, u[e]);
+    return;
+  }
+  void* kdst = part == 1 ? a.kspans[sp] : nullptr;
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < EPT; ++e)
+    if ((tid + e * NT) * 4 < n) {
+#pragma unroll
+      for (int x = 0; x < 4; ++x) ss = __builtin_fmaf(u[e][x], u[e][x], ss);
+    }
+  ss = wave_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  if (gamma) {
+    ss = 0.f;
+#pragma unroll
+    for (int w = 0; w < NT / 64; ++w) ss += red[w];
+    const float inv = 1.f / sqrtf(ss / (float)n + a.eps);
+#pragma unroll
+    for (int e = 0; e < EPT; ++e)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) u[e][x] = u[e][x] * inv * gm[e][x];
+  }
+  if (half && !a.pairs) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e)
+      if ((tid + e * NT) * 4 < n) *reinterpret_cast<f32x4_t*>(&us[c[e]]) = u[e];
+    __syncthreads();
+  }
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) {
+    if ((tid + e * NT) * 4 >= n) continue;
+    const int d0 = c[e] % a.D;
+    f32x4_t y = u[e];
+    if (d0 < a.rot_dims) {
+      if (a.pairs) {
+#pragma unroll
+        for (int x = 0; x < 4; x += 2)
+          if (d0 + x < a.rot_dims) {
+            const int p = (d0 + x) >> 1;
+            y[x] = u[e][x] * cs[p] - u[e][x + 1] * sn[p];
+            y[x + 1] = u[e][x + 1] * cs[p] + u[e][x] * sn[p];
+          }
+      } else {
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+          const int d = d0 + x;
+          if (d < half) y[x] = u[e][x] * cs[d] - us[c[e] + x + half] * sn[d];
+          else if (d < a.rot_dims) y[x] = u[e][x] * cs[d - half] + us[c[e] + x - half] * sn[d - half];
+        }
+      }
+    }
+    if (part == 0) *reinterpret_cast<f32x4_t*>(a.q_out + (size_t)t * a.ldq + c[e]) = y;
+    else store4(kdst, in_span * n + c[e], a.cdt, y);
+  }
+}
+
 // ------------------------------------------------------------------------------------------------ f32 row kernel
 struct GqaArgs {
-  float* out; long ldo;
+  void* out; int odt; long ldo;
   const float* q; long ldq;
   void* const* kspans; void* const* vspans; int span_stride, span_len;
   const void* sink; int wdt, sink_mode;   // 0: none, 1: sink[h], 2: the constant 0
@@ -257,7 +386,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(GqaArgs a) {
 #pragma unroll
       for (int v = 0; v < RV; ++v) {
         const int r = v * 64 + lane;
-        if (r < DV) a.out[(size_t)t * a.ldo + (size_t)hq * DV + r] = acc[v] / den * gt;
+        if (r < DV) st_any(a.out, (size_t)t * a.ldo + (size_t)hq * DV + r, a.odt, acc[v] / den * gt);
       }
     }
   }
@@ -473,10 +602,10 @@ __global__ __launch_bounds__(256) void gqa_attn_mc_kernel(GqaArgs a) {
   if (!row_ok) return;
   if (nsplit == 1) {
     const float inv = (a.gate ? a.gate[(size_t)(row0 + tq) * a.ldg + h] : 1.f) / l;
-    float* o = a.out + (size_t)(row0 + tq) * a.ldo + (size_t)hq * DV + kb * 4;
+    const size_t o = (size_t)(row0 + tq) * a.ldo + (size_t)hq * DV + kb * 4;
 #pragma unroll
     for (int t = 0; t < DT; ++t)
-      if (t * 16 + kb * 4 < DV) *reinterpret_cast<f32x4_t*>(o + t * 16) = f32x4_t{oacc[t][0] * inv, oacc[t][1] * inv, oacc[t][2] * inv, oacc[t][3] * inv};
+      if (t * 16 + kb * 4 < DV) store4(a.out, o + t * 16, a.odt, f32x4_t{oacc[t][0] * inv, oacc[t][1] * inv, oacc[t][2] * inv, oacc[t][3] * inv});
   } else {
     float* o = a.ws + ((size_t)split * a.rows_total + (size_t)(row0 + tq) * H * M + hq) * (Vp + 4);
 #pragma unroll
@@ -521,14 +650,14 @@ __device__ __forceinline__ float merge_splits(const float* __restrict__ base, si
 }
 
 // one workgroup per (row, query vector)
-__global__ __launch_bounds__(256) void gqa_attn_merge_kernel(float* __restrict__ out, long ldo, const float* __restrict__ ws, int nsplit,
+__global__ __launch_bounds__(256) void gqa_attn_merge_kernel(void* __restrict__ out, int odt, long ldo, const float* __restrict__ ws, int nsplit,
                                                              int rows_total, int H, int maps, int DV, int Vp, const float* __restrict__ gate, long ldg) {
   __shared__ float wgt[1024];
   __shared__ float red[4];
   const int gi = blockIdx.x, HQ = H * maps, t = gi / HQ, hq = gi - t * HQ, h = hq / maps;
   const size_t rec = (size_t)Vp + 4;
   const float v = merge_splits(ws + (size_t)gi * rec, (size_t)rows_total * rec, nsplit, Vp, DV, wgt, red);
-  if (threadIdx.x < DV) out[(size_t)t * ldo + (size_t)hq * DV + threadIdx.x] = v * (gate ? gate[(size_t)t * ldg + h] : 1.f);
+  if (threadIdx.x < DV) st_any(out, (size_t)t * ldo + (size_t)hq * DV + threadIdx.x, odt, v * (gate ? gate[(size_t)t * ldg + h] : 1.f));
 }
 
 // one workgroup per (row, head) of two maps: both merged, then d = first - lam * second, y = d / sqrt(mean(d^2) + eps) * out_scale
@@ -596,31 +725,51 @@ int dihip_qkv_conv_prep_append(void* stream, const float* x, long ld, const void
                  kspans, vspans, span_stride, span_len, cache_dtype, tok_slot, tok_pos, tok_off, H * D, G * D, G * DV, D};
   const size_t lds = (size_t)H * D * sizeof(float);      // (G <= H: the key row fits too)
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+  const auto al16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15u) == 0; };
+  const int C = (H + G) * D + G * DV, longest = H * D > G * DV ? H * D : G * DV;
+  if (D % 4 == 0 && DV % 4 == 0 && al16(x) && ld % 4 == 0 && al16(conv) && (!a.tail || al16(tail)) && al16(q_out) && ldq % 4 == 0 && (!qnorm || al16(qnorm)) &&
+      (!knorm || al16(knorm)) && C % 4 == 0 && longest <= 16384) {
+    auto go = [&](auto wt, auto nt, auto ept) {
+      constexpr int WT = decltype(wt)::value, NT = decltype(nt)::value, EPT = decltype(ept)::value;
+      hipLaunchKernelGGL((qkv_conv_prep_append_vec_kernel<WT, NT, EPT>), dim3(T, 3), dim3(NT), layout == 1 && rot_dims ? lds : 0, s, a);
+    };
+    auto by_n = [&](auto wt) {
+      using one = std::integral_constant<int, 1>;
+      if (longest <= 1024) go(wt, std::integral_constant<int, 256>{}, one{});
+      else if (longest <= 2048) go(wt, std::integral_constant<int, 512>{}, one{});
+      else if (longest <= 4096) go(wt, std::integral_constant<int, 1024>{}, one{});
+      else if (longest <= 8192) go(wt, std::integral_constant<int, 1024>{}, std::integral_constant<int, 2>{});
+      else go(wt, std::integral_constant<int, 1024>{}, std::integral_constant<int, 4>{});
+    };
+    if (w_dtype == DIHIP_F32) by_n(std::integral_constant<int, DIHIP_F32>{});
+    else by_n(std::integral_constant<int, DIHIP_BF16>{});
+    return launch_status();
+  }
   if (H * D <= 1024) hipLaunchKernelGGL(qkv_conv_prep_append_kernel<256>, dim3(T, 3), dim3(256), lds, s, a);
   else hipLaunchKernelGGL(qkv_conv_prep_append_kernel<1024>, dim3(T, 3), dim3(1024), lds, s, a);
   return launch_status();
 }
 
-static int gqa_check(const char* what, const float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
+static int gqa_check(const char* what, const void* out, int odt, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
                      int span_stride, int span_len, const void* sink, int w_dtype, int sink_mode, const float* gate, long ldg, int H, int G,
                      int D, int DV, int maps, int keep_first) {
   DIHIP_REQUIRE(maps >= 1 && maps <= 8 && keep_first >= 0, DIHIP_PARAM_ERROR, "%s: 1 to 8 maps per head, no negative count of kept keys", what);
   DIHIP_REQUIRE(out && q && kspans && vspans && span_stride > 0 && span_len > 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && DV > 0 &&
-                    ldo >= (long)H * maps * DV && ldq >= (long)H * maps * D && seq_dtype_ok(w_dtype), DIHIP_PARAM_ERROR, "%s: bad argument", what);
+                    ldo >= (long)H * maps * DV && ldq >= (long)H * maps * D && seq_dtype_ok(w_dtype) && seq_dtype_ok(odt), DIHIP_PARAM_ERROR, "%s: bad argument", what);
   DIHIP_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 1 || sink) && (!gate || ldg >= H || ldg == 0), DIHIP_PARAM_ERROR,
                 "%s: bad sink mode or gate", what);
   return DIHIP_SUCCESS;
 }
 
-int dihip_gqa_attn(void* stream, float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
+int dihip_gqa_attn(void* stream, void* out, int out_dtype, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
                    int span_stride, int span_len, int cache_dtype, const void* sink, int w_dtype, int sink_mode, float softcap,
                    const float* gate, long ldg, const int32_t* tok_slot, const int32_t* tok_pos, int T, int H, int G, int D, int DV,
                    float scale, int maps, int window, int keep_first) {
-  if (int rc = gqa_check("gqa_attn", out, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, gate, ldg, H, G, D, DV, maps, keep_first)) return rc;
+  if (int rc = gqa_check("gqa_attn", out, out_dtype, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, gate, ldg, H, G, D, DV, maps, keep_first)) return rc;
   DIHIP_REQUIRE(T >= 0 && tok_slot && tok_pos && seq_dtype_ok(cache_dtype), DIHIP_PARAM_ERROR, "gqa_attn: bad argument");
   DIHIP_REQUIRE(D <= 256 && DV <= 512, DIHIP_EXCEED_LIMIT_ERROR, "gqa_attn: head sizes above 256 (keys) / 512 (values)");
   if (T == 0) return DIHIP_SUCCESS;
-  GqaArgs a{out, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, softcap, gate, ldg, tok_slot, tok_pos,
+  GqaArgs a{out, out_dtype, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, softcap, gate, ldg, tok_slot, tok_pos,
             nullptr, nullptr, nullptr, H, G, D, DV, scale, nullptr, 0, maps, window, keep_first};
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   auto go = [&](auto ct, auto rv) {
@@ -646,12 +795,12 @@ size_t dihip_gqa_attn_mc_workspace_bytes(int T, int HQ, int DV, int nsplit) {
   return nsplit > 1 ? (size_t)nsplit * T * HQ * (((DV + 15) & ~15) + 4) * sizeof(float) : 0;
 }
 
-int dihip_gqa_attn_mc(void* stream, float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
+int dihip_gqa_attn_mc(void* stream, void* out, int out_dtype, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
                       int span_stride, int span_len, const void* sink, int w_dtype, int sink_mode, float softcap, const float* gate,
                       long ldg, const int32_t* tok_pos, const int32_t* ent_slot, const int32_t* ent_row0, const int32_t* ent_count, int E,
                       int max_count, int T, int H, int G, int D, int DV, float scale, int maps, int window, int keep_first, int nsplit,
                       void* ws, size_t ws_bytes, void* diff_out, int diff_dtype, long ldd, float lam, float out_scale, float eps) {
-  if (int rc = gqa_check("gqa_attn_mc", out, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, gate, ldg, H, G, D, DV, maps, keep_first)) return rc;
+  if (int rc = gqa_check("gqa_attn_mc", out, out_dtype, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, gate, ldg, H, G, D, DV, maps, keep_first)) return rc;
   DIHIP_REQUIRE(dihip_gqa_attn_mc_supported(D, DV, span_len, DIHIP_BF16), DIHIP_PARAM_ERROR,
                 "gqa_attn_mc: head sizes %d / %d (multiples of 8 up to 256 / 128) or span_len %d (a multiple of 32) not served", D, DV, span_len);
   DIHIP_REQUIRE(E >= 0 && T >= 0 && max_count >= 0 && tok_pos && ent_slot && ent_row0 && ent_count && ldo % 4 == 0 && ldq % 4 == 0,
@@ -659,13 +808,13 @@ int dihip_gqa_attn_mc(void* stream, float* out, long ldo, const float* q, long l
   DIHIP_REQUIRE((reinterpret_cast<uintptr_t>(out) & 15u) == 0 && (reinterpret_cast<uintptr_t>(q) & 15u) == 0, DIHIP_PARAM_ERROR,
                 "gqa_attn_mc: q / out must be 16-byte aligned");
   DIHIP_REQUIRE(nsplit >= 1 && nsplit <= 1024 && (long)E * G * maps <= 65535, DIHIP_PARAM_ERROR, "gqa_attn_mc: bad split / portion count");
-  DIHIP_REQUIRE(!diff_out || (maps == 2 && ldd >= (long)H * DV && seq_dtype_ok(diff_dtype)), DIHIP_PARAM_ERROR,
+  DIHIP_REQUIRE(!diff_out || (maps == 2 && out_dtype == DIHIP_F32 && ldd >= (long)H * DV && seq_dtype_ok(diff_dtype)), DIHIP_PARAM_ERROR,
                 "gqa_attn_mc: the difference of the maps needs two maps and rows of H * DV elements");
   DIHIP_REQUIRE(ws_bytes >= dihip_gqa_attn_mc_workspace_bytes(T, H * maps, DV, nsplit) && (nsplit == 1 || ws), DIHIP_PARAM_ERROR,
                 "gqa_attn_mc: workspace too small");
   if (E == 0 || max_count == 0) return DIHIP_SUCCESS;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  GqaArgs a{out, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, softcap, gate, ldg, nullptr, tok_pos,
+  GqaArgs a{out, out_dtype, ldo, q, ldq, kspans, vspans, span_stride, span_len, sink, w_dtype, sink_mode, softcap, gate, ldg, nullptr, tok_pos,
             ent_slot, ent_row0, ent_count, H, G, D, DV, scale, (float*)ws, T * H * maps, maps, window, keep_first};
   const int hpg = H / G, Dp = (D + 31) & ~31, Vp = (DV + 15) & ~15;
   const dim3 grid((unsigned)(((long)max_count * hpg + 63) / 64), E * G * maps, nsplit);
@@ -685,9 +834,9 @@ int dihip_gqa_attn_mc(void* stream, float* out, long ldo, const float* q, long l
     hipLaunchKernelGGL(gqa_attn_merge_diff_kernel, dim3(T * H), dim3(256), 0, s, diff_out, diff_dtype, ldd, (const float*)ws, nsplit, T * H * maps, H, DV,
                        Vp, gate, ldg, lam, out_scale, eps);
   else if (nsplit > 1)
-    hipLaunchKernelGGL(gqa_attn_merge_kernel, dim3(T * H * maps), dim3(256), 0, s, out, ldo, (const float*)ws, nsplit, T * H * maps, H, maps, DV, Vp, gate, ldg);
+    hipLaunchKernelGGL(gqa_attn_merge_kernel, dim3(T * H * maps), dim3(256), 0, s, out, out_dtype, ldo, (const float*)ws, nsplit, T * H * maps, H, maps, DV, Vp, gate, ldg);
   else if (diff_out)
-    hipLaunchKernelGGL(maps_diff_norm_kernel, dim3((unsigned)(((long)T * H + 3) / 4)), dim3(256), 0, s, diff_out, diff_dtype, ldd, out, ldo, lam, out_scale,
+    hipLaunchKernelGGL(maps_diff_norm_kernel, dim3((unsigned)(((long)T * H + 3) / 4)), dim3(256), 0, s, diff_out, diff_dtype, ldd, (const float*)out, ldo, lam, out_scale,
                        eps, T * H, H, DV);
   return launch_status();
 }

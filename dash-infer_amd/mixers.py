@@ -307,8 +307,8 @@ class GroupedQueryAttention:
         assert w["v"].shape[0] == self.G * vdim
         names = run_names(key, runs)
         if self.taps:
-            self.conv = torch.cat([w["q.conv"], w["k.conv"], w["v.conv"]], 0).contiguous()
-            assert self.conv.shape == (self.g_lo, self.taps)
+            self.conv = torch.cat([w["q.conv"], w["k.conv"], w["v.conv"]], 0).t().contiguous()      # [taps, channels]
+            assert self.conv.shape == (self.taps, self.g_lo)
             self.tails = [state.add_state(n + ".tail", (self.taps - 1, self.g_lo)) if self.taps > 1 else None for n in names]
         self.out_gain, self.out_scale = None, float(out_scale)
         if float(out_scale) != 1.0:      # a constant output gate: one row for all tokens
@@ -333,7 +333,7 @@ class GroupedQueryAttention:
         return so.linear(self.mix(ctx, a, run), self.o, self.o_b, math=ctx.math)
 
     def mix(self, ctx, a, run=0, out=None):
-        """a: the input product's rows -> what the output product reads.  out: rows of a wider f32 buffer (or None)"""
+        """a: the input product's rows -> what the output product reads.  out: rows of a wider buffer (or None)"""
         H, G, D, V = self.H, self.G, self.D, self.V
         ktable, vtable = self.ktables[run], self.vtables[run]
         assert out is None or (self.talk is None and self.differential is None)
@@ -357,6 +357,8 @@ class GroupedQueryAttention:
             o = so.talk_attn(a, ktable, vtable, ctx.tok_slot, ctx.tok_pos, ctx.max_pos, H, G, D, V, self.scale, self.talk, temp=self.head_temp,
                              gate=a[:, self.g_lo:] if self.elem_gate else None, window=self.window, out=ctx.act_buffer(H * V))
             return o
+        if out is None and self.differential is None:
+            out = ctx.act_buffer(H * V)
         if ctx.math == so.MATH_BF16 and self.mc:
             o = so.gqa_attn_mc(q, ktable, vtable, ctx.tok_pos, ctx.ent_slot, ctx.ent_row0, ctx.ent_count, ctx.max_count, ctx.max_pos,
                                H, G, D, V, self.scale, self.sink, self.sink_mode, self.softcap, gate, out=out, maps=self.maps, window=self.window,
@@ -492,7 +494,7 @@ class WeightedPair:
     def rows(self, ctx, h, h16=None, run=0):
         """-> the output product's rows without `bias`, which a residual step adds (seq_ops.residual_rmsnorm)"""
         a = so.linear(h16 if h16 is not None else h, self.w_in, self.b_in, act="sigmoid" if self.act_cols else None, act_cols=self.act_cols, math=ctx.math)
-        both = torch.empty(ctx.T, self.o.shape[1], dtype=torch.float32, device=a.device)
+        both = ctx.act_buffer(self.o.shape[1])
         self.left.mix(ctx, a[:, : self.r_lo], run, out=both[:, : self.k_left])
         self.right.mix(ctx, a[:, self.r_lo:], run, out=both[:, self.k_left:])
         return so.linear(both, self.o, math=ctx.math)
@@ -583,16 +585,24 @@ class ExpertMlp:
                 self.b_x = None
 
     def parts(self, ctx, h, h16=None):
-        """-> ((rows, dst, wts), the gated shared expert's rows or None): what the residual step sums (seq_ops.residual_rmsnorm).  Router,
-        shared gate and the shared expert's first product are ONE product: its sums are f32 either way."""
+        """-> ((rows, dst, wts), the gated shared expert's rows or None): what the residual step sums (seq_ops.residual_rmsnorm).  For few
+        rows the router, the shared gate and the shared expert's first product are ONE product (its sums are f32 either way); many rows
+        keep the few columns out of the matrix-core tiles."""
         x = h16 if h16 is not None else h
         if self.w_x is None:
             assert self.shared is None and not self.identity
             return self.__call__(ctx, h, h16, defer=True), None
-        z = so.linear(x, self.w_x, self.b_x, act="sigmoid", act_cols=(self.sg_lo, self.sg_lo + 1), math=ctx.math)
+        gate = dict(act="sigmoid", act_cols=(self.sg_lo, self.sg_lo + 1))
+        if ctx.T <= 16 or self.gu_lo > 64:
+            z = so.linear(x, self.w_x, self.b_x, math=ctx.math, **gate)
+            gu = z[:, self.gu_lo:]
+        else:
+            n = self.gu_lo
+            z = so.linear(x, self.w_x[:n], self.b_x[:n] if self.b_x is not None else None, math=so.MATH_F32 if ctx.math == so.MATH_F32 else so.MATH_F32_STREAM, **gate)
+            gu = so.linear(x, self.w_x[n:], math=ctx.math)
         routed = self._routed(ctx, x, z[:, : self.router.shape[0]])
         F = self.shared.F
-        g = so.moe_glu(z[:, self.gu_lo:], F, self.shared.limit, GLU_SLOPE, ctx.act_buffer(F))
+        g = so.moe_glu(gu, F, self.shared.limit, GLU_SLOPE, ctx.act_buffer(F))
         return routed[1:], so.linear(g, self.shared.down, mul=z[:, self.sg_lo: self.sg_lo + 1], mul_group=True, math=ctx.math)
 
     def __call__(self, ctx, h, h16=None, defer=False):

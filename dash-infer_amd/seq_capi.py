@@ -40,12 +40,12 @@ _SIGS = {
     "dihip_add_dyt": (i32, [vp, vp, vp, vp, lng, vp, lng, vp, f32, vp, vp, i32, vp, vp, i32, i32]),
     "dihip_qkv_prep_append": (i32, [vp, vp, lng, i32, i32, i32, i32, i32, i32, i32, i32, vp, vp, i32, f32, vp, i32, i32, f32, f32, vp, vp, lng, vp, vp,
                                     i32, i32, i32, vp, vp, i32]),
-    "dihip_gqa_attn": (i32, [vp, vp, lng, vp, lng, vp, vp, i32, i32, i32, vp, i32, i32, f32, vp, lng, vp, vp, i32, i32, i32, i32, i32, f32, i32, i32,
+    "dihip_gqa_attn": (i32, [vp, vp, i32, lng, vp, lng, vp, vp, i32, i32, i32, vp, i32, i32, f32, vp, lng, vp, vp, i32, i32, i32, i32, i32, f32, i32, i32,
                              i32]),
     "dihip_maps_diff_norm": (i32, [vp, vp, i32, lng, vp, lng, f32, f32, f32, i32, i32, i32]),
     "dihip_gqa_attn_mc_supported": (i32, [i32, i32, i32, i32]),
     "dihip_gqa_attn_mc_workspace_bytes": (sz, [i32, i32, i32, i32]),
-    "dihip_gqa_attn_mc": (i32, [vp, vp, lng, vp, lng, vp, vp, i32, i32, vp, i32, i32, f32, vp, lng, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32,
+    "dihip_gqa_attn_mc": (i32, [vp, vp, i32, lng, vp, lng, vp, vp, i32, i32, vp, i32, i32, f32, vp, lng, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32,
                                 i32, f32, i32, i32, i32, i32, vp, sz, vp, i32, lng, f32, f32, f32]),
     "dihip_gla_workspace_bytes": (sz, [i32, i32, i32, i32, i32, i32, i32]),
     "dihip_gla": (i32, [vp, vp, lng, vp, lng, vp, lng, vp, lng, vp, lng, f32, f32, vp, vp, vp, vp, i32, i32, i32, i32, i32, i32, i32, vp, sz]),

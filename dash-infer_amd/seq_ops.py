@@ -249,11 +249,11 @@ def qkv_prep_append(a, q_off, k_off, v_off, H, G, D, DV, qnorm, knorm, eps, freq
 
 
 def qkv_conv_prep_append(x, conv, tail, one_row, H, G, D, DV, qnorm, knorm, eps, freq, rot_dims, layout, mag, ktable, vtable, tok_slot, tok_pos, tok_off):
-    """short convolution on every channel of x = [q | k | v] (f32 rows), norms over the whole query / key row, rotation, append of k and v to
+    """short convolution (conv [taps, channels]) on every channel of x = [q | k | v] (f32 rows), norms over the whole query / key row, rotation, append of k and v to
     their pages; one_row: every portion of the step has one row (its tail moves on here) -> the queries, f32 [T, H * D]"""
-    T, taps = x.shape[0], conv.shape[1]
+    T, taps = x.shape[0], conv.shape[0]
     C = (H + G) * D + G * DV
-    assert x.dtype == torch.float32 and x.shape[1] >= C and conv.shape == (C, taps) and conv.is_contiguous() and ktable.dtype == vtable.dtype
+    assert x.dtype == torch.float32 and x.shape[1] >= C and conv.shape == (taps, C) and conv.is_contiguous() and ktable.dtype == vtable.dtype
     assert ktable.row_elems == G * D and vtable.row_elems == G * DV and (taps == 1 or (tail.shape[1:] == (taps - 1, C) and tail.is_contiguous()))
     assert (qnorm is None or qnorm.shape == (H * D,)) and (knorm is None or knorm.shape == (G * D,))
     assert all(w is None or w.dtype == conv.dtype for w in (qnorm, knorm))
@@ -272,10 +272,10 @@ SINK_NONE, SINK_PER_HEAD, SINK_ZERO = 0, 1, 2
 def gqa_attn(q, ktable, vtable, tok_slot, tok_pos, H, G, D, DV, scale, sink=None, sink_mode=SINK_NONE, softcap=0.0, gate=None, out=None,
              maps=1, window=0, keep_first=0):
     """q: f32 [T, >= H * maps * D] rows (a column slice is fine); gate: f32 [T, >= H] or None -> f32 [T, H * maps * DV].  window > 0:
-    a row reads the keys less than `window` positions back and the first keep_first keys of its sequence"""
+    a row reads the keys less than `window` positions back and the first keep_first keys of its sequence.  out: f32 or bf16 rows"""
     T = q.shape[0]
     o = out if out is not None else torch.empty(T, H * maps * DV, dtype=torch.float32, device=q.device)
-    check(lib().dihip_gqa_attn(stream(), ptr(o), _rows(o), ptr(q), _rows(q), ptr(ktable.ptrs), ptr(vtable.ptrs), ktable.max_spans, ktable.span_len,
+    check(lib().dihip_gqa_attn(stream(), ptr(o), dt(o), _rows(o), ptr(q), _rows(q), ptr(ktable.ptrs), ptr(vtable.ptrs), ktable.max_spans, ktable.span_len,
                                _DT[ktable.dtype], ptr(sink), dt(sink) if sink is not None else F32_CODE, int(sink_mode), float(softcap or 0.0),
                                ptr(gate), _rows(gate) if gate is not None else 0, ptr(tok_slot), ptr(tok_pos), T, H, G, D, DV, float(scale),
                                int(maps), int(window or 0), int(keep_first or 0)), "dihip_gqa_attn")
@@ -302,7 +302,7 @@ def gqa_attn_mc(q, ktable, vtable, tok_pos, ent_slot, ent_row0, ent_count, max_c
     ws = None
     if nsplit > 1:
         ws = torch.empty(int(lib().dihip_gqa_attn_mc_workspace_bytes(T, H * maps, DV, nsplit)), dtype=torch.uint8, device=q.device)
-    check(lib().dihip_gqa_attn_mc(stream(), ptr(o), _rows(o), ptr(q), _rows(q), ptr(ktable.ptrs), ptr(vtable.ptrs), ktable.max_spans,
+    check(lib().dihip_gqa_attn_mc(stream(), ptr(o), dt(o), _rows(o), ptr(q), _rows(q), ptr(ktable.ptrs), ptr(vtable.ptrs), ktable.max_spans,
                                   ktable.span_len, ptr(sink), dt(sink) if sink is not None else F32_CODE, int(sink_mode), float(softcap or 0.0),
                                   ptr(gate), _rows(gate) if gate is not None else 0, ptr(tok_pos), ptr(ent_slot), ptr(ent_row0), ptr(ent_count),
                                   E, int(max_count), T, H, G, D, DV, float(scale), int(maps), window, keep_first, int(nsplit), ptr(ws),

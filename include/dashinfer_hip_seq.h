@@ -149,7 +149,8 @@ int dihip_qkv_prep_append(void* stream, float* qkv, long ld, int q_off, int k_of
                           const int32_t* tok_slot, const int32_t* tok_pos, int T);
 
 /* step 1 of a layer with short convolutions: per channel c of x[t] = [q [H, D] | k [G, D] | v [G, DV]] (f32)
- *   u[t, c] = sum_{j < taps} conv[c, j] * x[t - (taps - 1) + j, c]   (earlier steps' inputs: tail, as dihip_causal_conv_state has it),
+ *   u[t, c] = sum_{j < taps} conv[j, c] * x[t - (taps - 1) + j, c]   (conv [taps][channels]; earlier steps' inputs: tail, as
+ *   dihip_causal_conv_state has it),
  * then the whole query row and the whole key row are divided by their root mean square and scaled by qnorm [H * D] / knorm [G * D]
  * (NULL: no norm), rotated per head as above; queries go to q_out, keys and values to their pages.  write_tail: every portion of the step
  * has one row, the tail is moved on here (else: dihip_conv_tail_update afterwards). */
@@ -164,8 +165,8 @@ int dihip_qkv_conv_prep_append(void* stream, const float* x, long ld, const void
  *   p = softmax over {s_j} and, with sink_mode 1 / 2, one more logit sink[h] / 0 that has no value
  *   out[t, h, m] = gate[t, h] * sum_j p_j v_j   (gate NULL: 1; ldg 0: one row [H] for every t)
  * for every map m < maps of the head (each a softmax of its own over the same values).
- * q [T, H, maps, D], out [T, H, maps, DV] f32.  Every product and sum in f32. */
-int dihip_gqa_attn(void* stream, float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
+ * q [T, H, maps, D] f32, out [T, H, maps, DV] of out_dtype.  Every product and sum in f32. */
+int dihip_gqa_attn(void* stream, void* out, int out_dtype, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
                    int span_stride, int span_len, int cache_dtype, const void* sink, int w_dtype, int sink_mode, float softcap,
                    const float* gate, long ldg, const int32_t* tok_slot, const int32_t* tok_pos, int T, int H, int G, int D,
                    int DV, float scale, int maps, int window, int keep_first);
@@ -175,7 +176,7 @@ int dihip_gqa_attn(void* stream, float* out, long ldo, const float* q, long ldq,
  * split walk, else as a launch of its own; `out` is then scratch. */
 int dihip_gqa_attn_mc_supported(int D, int DV, int span_len, int cache_dtype);
 size_t dihip_gqa_attn_mc_workspace_bytes(int T, int H_times_maps, int DV, int nsplit);
-int dihip_gqa_attn_mc(void* stream, float* out, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
+int dihip_gqa_attn_mc(void* stream, void* out, int out_dtype, long ldo, const float* q, long ldq, void* const* kspans, void* const* vspans,
                       int span_stride, int span_len, const void* sink, int w_dtype, int sink_mode, float softcap,
                       const float* gate, long ldg, const int32_t* tok_pos, const int32_t* ent_slot, const int32_t* ent_row0,
                       const int32_t* ent_count, int E, int max_count, int T, int H, int G, int D, int DV, float scale,

@@ -506,6 +506,38 @@ class WeightedPair:
         return y
 
 
+class StateSpaceMixer:
+    def __init__(self, key, heads, vdim, n_state, groups, taps, norm_groups, w, state):
+        """w: in [2*inner + 2*groups*n_state + heads, width] laid out [z | x | B | C | dt] (inner = heads*vdim), conv [inner +
+        2*groups*n_state, taps] + conv.b over [x | B | C], dt_bias / A_log / D [heads], norm [inner], o [width, inner].
+        Per head (head h reads group h / (heads / groups)):  step = softplus(dt + dt_bias);  S <- exp(-exp(A_log) step) S + step B x^T;
+        y = S^T C + D x;  out = o . (rms-norm over norm_groups parts of (y * silu(z)) * norm)."""
+        assert heads % groups == 0 and (heads * vdim) % norm_groups == 0
+        self.H, self.P, self.N, self.G, self.taps, self.norm_groups = heads, vdim, n_state, groups, int(taps), int(norm_groups)
+        self.inner, self.ch = heads * vdim, heads * vdim + 2 * groups * n_state
+        self.w_in = w["in"].contiguous()
+        assert self.w_in.shape[0] == self.inner + self.ch + heads and w["conv"].shape == (self.ch, self.taps)
+        self.conv, self.conv_b = w["conv"].contiguous(), w["conv.b"].contiguous()
+        self.dt_bias, self.a_log, self.skip = w["dt_bias"].contiguous(), w["A_log"].contiguous(), w["D"].contiguous()
+        self.norm, self.o = w["norm"].contiguous(), w["o"].contiguous()
+        assert self.norm.shape[0] == self.inner and self.o.shape[1] == self.inner
+        self.S = state.add_state(key + ".S", (heads, n_state, vdim))
+        self.tail = state.add_state(key + ".tail", (self.taps - 1, self.ch)) if self.taps > 1 else None
+
+    def __call__(self, ctx, h, h16=None):
+        inner, ch, GN = self.inner, self.ch, self.G * self.N
+        a = so.linear(h16 if h16 is not None else h, self.w_in, math=ctx.math)                    # [z | x B C | dt], f32
+        z, xbc, dtr = a[:, :inner], a[:, inner: inner + ch], a[:, inner + ch:]
+        u = so.causal_conv_state(xbc, self.conv, self.conv_b, self.tail, ctx.tok_slot, ctx.tok_off, act="silu")
+        if self.tail is not None:
+            so.conv_tail_update(self.tail, xbc, self.taps, ctx.ent_slot, ctx.ent_row0, ctx.ent_count)
+        y = so.ssd(u, u[:, inner: inner + GN], u[:, inner + GN:], dtr, self.dt_bias, self.a_log, self.S, ctx.ent_slot, ctx.ent_row0,
+                   ctx.ent_count, ctx.max_count, self.H, self.G, self.N, self.P)
+        yn = so.gate_group_rmsnorm(y, z, self.norm, ctx.eps, self.H, self.P, self.norm_groups, x=u, skip=self.skip,
+                                   out=ctx.act_buffer(inner))
+        return so.linear(yn, self.o, math=ctx.math)
+
+
 class SideBySide:
     """two mixers that read the same input: coef * (rms_norm(left) * w_left + rms_norm(right) * w_right), norms over the width"""
 

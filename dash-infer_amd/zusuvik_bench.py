@@ -3,6 +3,7 @@ resemble real models', per-operator times of the design's kernels against their 
 active feed-forward size (the closest design the engine serves: parallel layers, grouped-query attention with capped scores, gated linear
 attention, routed clamped units) with their like operators beside them."""
 import math
+import sys
 
 import torch
 
@@ -184,8 +185,16 @@ def operator_table(size, prompt_len):
         def vogusun_two():
             so.linear(h16, rb, out=logits, math=so.MATH_F32_STREAM)
             so.linear(h16, wv, out=zv, math=so.MATH_BF16)
-        add(f"router + shared gate + shared [gate | up] in one product, {wx.shape[0]} columns", T, lambda: so.linear(h16, wx, out=zx, math=so.MATH_BF16),
-            *lin(wx.shape[0], W, 2.0), like=("router logits; a dense [gate | up] product", vogusun_two, *lin(2 * FS + E, W, 2.0)))
+        few = ((E + 3) & ~3) + 4
+        zr = torch.empty(T, few, device=dev)
+
+        def zusuvik_x():       # few rows: one product; many: the few columns apart
+            if T <= 16:
+                return so.linear(h16, wx, out=zx, math=so.MATH_BF16)
+            so.linear(h16, wx[:few], out=zr, math=so.MATH_F32_STREAM)
+            so.linear(h16, wx[few:], out=zv, math=so.MATH_BF16)
+        add(f"router, shared gate and shared [gate | up], {wx.shape[0]} columns", T, zusuvik_x, *lin(wx.shape[0], W, 2.0),
+            like=("router logits; a dense [gate | up] product", vogusun_two, *lin(2 * FS + E, W, 2.0)))
         w_gu, w_dn, used = bf(E, 2 * F, W), bf(E, W, F), min(E, R)
         gu, y = torch.empty(R, 2 * F, device=dev), torch.empty(R, F, dtype=torch.bfloat16, device=dev)
         add(f"routing: top-{top} of {E}, grouping by expert", T, lambda: so.moe_route(logits, top), 4.0 * T * E + 16.0 * R)
@@ -219,7 +228,6 @@ def run(args):
             entry[name]["weight_bytes"] = int(sum(v.numel() * v.element_size() for k, v in t.items() if k != "embed" or "head" not in t))
             del eng, t
             torch.cuda.empty_cache()
-            import sys
             print(f"# {size} {name} {entry[name]}", file=sys.stderr, flush=True)
         entry["operators"] = operator_table(size, prompt_len)
         res["sizes"][size] = entry

@@ -55,7 +55,7 @@ def random_model(size, device="cuda", seed=0, pattern=PATTERN, loop=None):
             for n, rows in (("q", H * D), ("k", H * D), ("v", H * V), ("g", H * V), ("i", H), ("f", H)):
                 t[q + f"right.{n}"] = r(rows, W)
             t[q + "right.o"], t[q + "right.norm"], t[q + "right.i.b"], t[q + "right.f.b"] = r(W, H * V), one(H * V), r(H, sd=1.0), 4 + r(H, sd=1.0)
-            m = {"left": left, "right": {"heads": H, "dim": D, "vdim": V, "gate_cap": 15.0}, "left_scale": 0.8, "right_scale": 0.6}
+            m = {"left": left, "right": {"heads": H, "dim": D, "vdim": V, "gate_cap": 15.0}, "left_scale": 0.75, "right_scale": 0.6}
         E, F, FS = s["experts"], s["expert_ff"], s["shared_ff"]
         for e, f in [(f"e{e}", F) for e in range(E)] + [("shared", FS)]:
             t[p + f"mlp.{e}.gate"], t[p + f"mlp.{e}.up"], t[p + f"mlp.{e}.down"] = r(f, W), r(f, W), r(W, f)

@@ -228,7 +228,7 @@ ATTENTION_SHAPES = {
     "plain": {},
     "odd_one_kv_head": dict(heads=3, kv_heads=1, dim=10, vdim=7, rot_dims=6, conv=2, scaling=None, softcap=3.0),
     "one_tap": dict(heads=4, kv_heads=4, dim=32, vdim=64, rot_dims=32, conv=1, scale=0.3),
-    "many_taps": dict(heads=2, kv_heads=2, dim=96, vdim=96, rot_dims=24, conv=7, scaling=dict(factor=2.0, low=1.0, high=4.0, original=256)),
+    "many_taps": dict(heads=2, kv_heads=2, dim=88, vdim=104, rot_dims=20, conv=7, scaling=dict(factor=2.0, low=1.0, high=4.0, original=256)),
     "wide_rows": dict(heads=10, kv_heads=5, dim=128, vdim=16, rot_dims=128, conv=3),
     "no_rotation_no_cap": dict(heads=1, kv_heads=1, dim=9, vdim=200, rot_dims=0, softcap=None),
 }

@@ -538,8 +538,8 @@ using namespace dihip;
 
 static size_t decay_gate_floats(int T, int H) { return ((size_t)3 * T * H + 3) & ~(size_t)3; }
 
-static int decay_run(const char* what, hipStream_t s, DecayArgs a, int T, int E, int max_count, int chunked, int k_off_for_rope, float* rope_rows, long rope_ld,
-                     int q_off, void* ws, size_t ws_bytes) {
+// rope_rows: the rows that hold q and k at q_off and k_off (chunked retention rotates them in place first; NULL: no rotation)
+static int decay_run(hipStream_t s, DecayArgs a, int T, int E, int max_count, int chunked, float* rope_rows, long rope_ld, int q_off, int k_off, void* ws) {
   const int H = a.H, D = a.D, DV = a.DV, cbs64 = (DV + 63) / 64;
   if (!chunked) {
     const size_t lds = (size_t)RB * a.rot_dims * sizeof(float);
@@ -564,7 +564,7 @@ static int decay_run(const char* what, hipStream_t s, DecayArgs a, int T, int E,
   a.ws = w;
   if (a.rot_dims) {
     const int work = 2 * H * (a.rot_dims >> 1);
-    hipLaunchKernelGGL(rope_rows_kernel, dim3(T, T >= 256 ? 1 : (work + 255) / 256), dim3(256), 0, s, rope_rows, rope_ld, q_off, H, k_off_for_rope, H, D, a.rot_dims,
+    hipLaunchKernelGGL(rope_rows_kernel, dim3(T, T >= 256 ? 1 : (work + 255) / 256), dim3(256), 0, s, rope_rows, rope_ld, q_off, H, k_off, H, D, a.rot_dims,
                        a.pairs, a.freq, a.tok_pos);
   }
   const auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15u) == 0; };
@@ -584,7 +584,6 @@ static int decay_run(const char* what, hipStream_t s, DecayArgs a, int T, int E,
   };
   if (vec) by_v(std::true_type{});
   else by_v(std::false_type{});
-  (void)what; (void)ws_bytes;
   return launch_status();
 }
 
@@ -622,7 +621,7 @@ int dihip_retention(void* stream, float* out, long ldo, float* rows, long ld, in
   a.freq = freq; a.rot_dims = rot_dims; a.pairs = layout == 0; a.tok_pos = tok_pos;
   a.S = state; a.ent_slot = ent_slot; a.ent_row0 = ent_row0; a.ent_count = ent_count;
   a.H = H; a.D = D; a.DV = DV;
-  return decay_run("retention", reinterpret_cast<hipStream_t>(stream), a, T, E, max_count, chunked, k_off, rows, ld, q_off, ws, ws_bytes);
+  return decay_run(reinterpret_cast<hipStream_t>(stream), a, T, E, max_count, chunked, rows, ld, q_off, k_off, ws);
 }
 
 int dihip_matrix_memory(void* stream, float* out, long ldo, float* den, const float* q, long ldq, const float* k, long ldk, const float* v, long ldv,
@@ -643,7 +642,7 @@ int dihip_matrix_memory(void* stream, float* out, long ldo, float* den, const fl
   a.S = state_s; a.N = state_n; a.M = state_m; a.mcopies = m_copies;
   a.ent_slot = ent_slot; a.ent_row0 = ent_row0; a.ent_count = ent_count;
   a.H = H; a.D = D; a.DV = DV;
-  return decay_run("matrix_memory", reinterpret_cast<hipStream_t>(stream), a, T, E, max_count, chunked, 0, nullptr, 0, 0, ws, ws_bytes);
+  return decay_run(reinterpret_cast<hipStream_t>(stream), a, T, E, max_count, chunked, nullptr, 0, 0, 0, ws);
 }
 
 }  // extern "C"
